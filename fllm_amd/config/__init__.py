@@ -4,6 +4,8 @@ from .dumizen import DumizenConfig
 from .llama import LlamaConfig, RopeScaling
 from .menitar import MenitarConfig
 from .purivik import PurivikConfig
+from .venadra import VenadraConfig
+from .zoguzen import ZoguzenConfig
 
 __all__ = ["ConfigError", "LayerSpec", "ModelSpec", "PartSpec", "RunEntry", "default_run_order",
-           "DumizenConfig", "LlamaConfig", "MenitarConfig", "PurivikConfig", "RopeScaling", "read_config_json"]
+           "DumizenConfig", "LlamaConfig", "MenitarConfig", "PurivikConfig", "RopeScaling", "VenadraConfig", "ZoguzenConfig", "read_config_json"]

@@ -1,5 +1,5 @@
-from . import (attention, block, conv_input, embedding, experts, lightning, mlp, norm, normed_attention, pair, rope, sigmoid_attention,
-               stream, talking_attention)  # noqa: F401  (register the parts)
+from . import (attention, block, conv_attention, conv_input, embedding, experts, gated_linear, lightning, min_gru, mlp, norm,
+               normed_attention, pair, rope, sigmoid_attention, stream, talking_attention, token_side)  # noqa: F401  (register the parts)
 from .base import Block, FeedForward, KVNeed, Mixer, Norm, Part, StateNeed
 from .runtime import Runtime
 

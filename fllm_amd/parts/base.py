@@ -61,6 +61,11 @@ import torch
 
 from ..config.spec import PartSpec
 
+class SizeFromFile(int):
+    """A size in `tensor_shapes` that only the checkpoint's tensor gives: any size fits there.  The number is what
+    random-weights mode uses."""
+
+
 # how random-weights mode fills a tensor
 INIT_MATRIX = "matrix"     # N(0, 0.02)
 INIT_NORM = "norm"         # 1 + U(-0.1, 0.1)
@@ -159,6 +164,13 @@ class Norm(Part):
 
     def forward(self, ctx, x, out=None, rows=None):
         raise NotImplementedError
+
+    def row_form(self):
+        """(weight, eps, centered) if the norm is (x - mean) * rsqrt(mean((x - mean)^2) + eps) * weight over a row, with the mean
+        taken off (`centered`, a layer norm) or taken as zero (an RMS norm); None if it is anything else.  For kernels that norm
+        a row they have just finished, or one row with several weights at once."""
+        prologue = self.fused_prologue()
+        return None if prologue is None else (prologue[0], prologue[1], False)
 
     def fused_prologue(self):
         """(scale, eps) if the norm is x * rsqrt(mean(x^2) + eps) * scale with a float32 device vector `scale`,

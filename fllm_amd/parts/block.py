@@ -1,6 +1,7 @@
 """Arrangement of parts in a layer.  `prenorm`: x += mixer(norm(x)); x += feed_forward(norm(x))
 (rust/engine/src/rust_decoder.rs:8764-8766, :9059-9088).  `parallel`: x += mixer(norm_a(x)) + feed_forward(norm_b(x)),
-both branches behind norms of their own of the same x.  `sandwich`: a norm before and a norm behind each part,
+both branches behind norms of their own of the same x, then, where the layer names one, a part of role `stream` that changes
+the sum (`extras["after"]`).  `sandwich`: a norm before and a norm behind each part,
 x += m * s_a * norm_a'(mixer(norm_a(x))); x += m * s_b * norm_b'(feed_forward(norm_b(x))), with a constant m and
 learned vectors s (a scale a lane of each branch)."""
 from __future__ import annotations
@@ -93,16 +94,23 @@ class PreNormBlock(Block):
 
 class ParallelBlock(Block):
     """Both branches read the stream as the layer found it, each through its own norm; their outputs are added to it.
-    Where both norms are of the form x * rsqrt(mean x^2 + eps) * w they share one pass over the rows."""
+    Where both norms are RMS norms, or both layer norms, with a weight a lane they share one pass over the rows."""
 
-    def __init__(self, spec, weights, rt, mixer=None, feed_forward=None, norms=None):
+    def __init__(self, spec, weights, rt, mixer=None, feed_forward=None, norms=None, extras=None):
         super().__init__(spec, weights, rt)
+        self.extras = dict(extras or {})
+        self.after = self.extras.get("after")
         self.mixer = mixer
         self.feed_forward = feed_forward
         self.mixer_norm = norms["mixer"]
         self.feed_forward_norm = norms["feed_forward"] if feed_forward is not None else None
 
     def forward(self, ctx, residual, binding):
+        self._both(ctx, residual, binding)
+        if self.after is not None:
+            self.after.forward(ctx, residual, None)
+
+    def _both(self, ctx, residual, binding):
         rt, ops = self.rt, self.rt.ops
         ctx.then_norm = ctx.prepared = None          # the sums of this block's parts are not read by a norm they know
         # a part may read the stream through its norm in one kernel with its first product, and add to it later: every
@@ -119,12 +127,13 @@ class ParallelBlock(Block):
         begun = begin(ctx, residual, self.feed_forward_norm) if begin is not None else None
         h_mixer = h_ff = None
         if projected is None and begun is None:
-            first = getattr(self.mixer_norm, "fused_prologue", lambda: None)()
-            second = getattr(self.feed_forward_norm, "fused_prologue", lambda: None)()
-            pair = getattr(ops, "rmsnorm_pair", None)
-            if pair is not None and first is not None and second is not None:
-                h_mixer, h_ff = rt.empty(tuple(residual.shape)), rt.empty(tuple(residual.shape))
-                pair(residual, first[0], first[1], h_mixer, second[0], second[1], h_ff)
+            first = getattr(self.mixer_norm, "row_form", lambda: None)()
+            second = getattr(self.feed_forward_norm, "row_form", lambda: None)()
+            if first is not None and second is not None and first[2] == second[2]:
+                pair = getattr(ops, "layernorm_pair" if first[2] else "rmsnorm_pair", None)
+                if pair is not None:
+                    h_mixer, h_ff = rt.empty(tuple(residual.shape)), rt.empty(tuple(residual.shape))
+                    pair(residual, first[0], first[1], h_mixer, second[0], second[1], h_ff)
         if projected is None and h_mixer is None:
             h_mixer = self.mixer_norm.forward(ctx, residual)
         if begun is None and h_ff is None:

@@ -4,6 +4,9 @@ conv(h)_t = sum_j w[:, j] * h_(t - taps + 1 + j) on every channel, zeros before 
 `ConvInput` wraps any mixer (`inner`: the wrapped mixer's PartSpec): it keeps the last taps - 1 inputs of every live request
 in a state of its own beside whatever the wrapped mixer keeps, convolves, and hands the result on.  Cache, state, portions
 and graphs are the wrapped mixer's; its tensors are listed under `inner.<name>`.
+
+`form` "shift": the mixer reads h + (h' - h) * shift, h' the previous token's h and `shift` one learned number a lane: the same
+convolution with the two taps (shift, -shift).
 """
 from __future__ import annotations
 
@@ -12,7 +15,7 @@ from types import SimpleNamespace
 import torch
 
 from ..registry import part_class, register_part
-from .base import INIT_MATRIX, Mixer, StateNeed, take_prepared
+from .base import INIT_MATRIX, INIT_NORM, Mixer, StateNeed, take_prepared
 
 _TAIL = "conv_inputs"      # the name of the wrapper's own state
 
@@ -21,7 +24,10 @@ class ConvInput(Mixer):
     @classmethod
     def tensor_shapes(cls, spec):
         inner = spec["inner"]
-        shapes = {"conv": ((spec["size"], spec["taps"]), INIT_MATRIX)}
+        if spec.get("form", "conv") == "shift":
+            shapes = {"shift": ((spec["size"],), INIT_NORM)}
+        else:
+            shapes = {"conv": ((spec["size"], spec["taps"]), INIT_MATRIX)}
         for name, shape in part_class("mixer", inner.kind).tensor_shapes(inner).items():
             shapes["inner." + name] = shape
         return shapes
@@ -29,10 +35,17 @@ class ConvInput(Mixer):
     def __init__(self, spec, weights, rt):
         super().__init__(spec, weights, rt)
         self.size = int(spec["size"])
-        self.taps = int(spec["taps"])
+        form = spec.get("form", "conv")
+        if form not in ("conv", "shift"):
+            raise ValueError(f"form {form!r}: 'conv' or 'shift'")
+        self.taps = 2 if form == "shift" else int(spec["taps"])
         if not 1 <= self.taps <= 16:
             raise ValueError(f"a convolution of {self.taps} taps is outside 1..16")
-        self.w = rt.vector(weights["conv"])                   # float32 [size, taps]
+        if form == "shift":
+            amount = rt.vector(weights["shift"])
+            self.w = torch.stack([amount, -amount], dim=1).contiguous()
+        else:
+            self.w = rt.vector(weights["conv"])               # float32 [size, taps]
         inner = spec["inner"]
         own = {name[len("inner."):]: t for name, t in weights.items() if name.startswith("inner.")}
         self.inner = part_class("mixer", inner.kind)(inner, own, rt)

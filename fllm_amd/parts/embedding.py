@@ -38,6 +38,7 @@ class LinearHead(Part):
         self.weight = rt.matrix(weights["weight"])
         self.vocab = int(spec["vocab_size"])
         self.scale = float(spec.get("scale", 1.0))       # logits = (W h) * scale, the product in float32
+        self.softcap = float(spec.get("softcap") or 0.0)      # then softcap * tanh(logits / softcap); 0: none
         rt.tile_for_decode(self.weight, priority=2)      # read once a step of up to 16 rows: after the layers' copies
 
     def forward(self, ctx, h):
@@ -45,6 +46,8 @@ class LinearHead(Part):
         self.rt.ops.linear(h, self.weight, logits)
         if self.scale != 1.0:
             self.rt.ops.scale_(logits, self.scale)
+        if self.softcap > 0.0:
+            self.rt.ops.softcap_(logits, self.softcap)
         return logits
 
 

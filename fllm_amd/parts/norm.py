@@ -57,5 +57,31 @@ class ScalarRMSNorm(RMSNorm):
         self.weight = rt.vector(g).reshape(1).expand(self.size).contiguous()
 
 
+class LayerNorm(Norm):
+    """y = (x - mean) / sqrt(mean((x - mean)^2) + eps) * w, in float32: the mean taken off first, no bias."""
+
+    @classmethod
+    def tensor_shapes(cls, spec):
+        return {"weight": ((spec["size"],), INIT_NORM)}
+
+    def __init__(self, spec, weights, rt):
+        super().__init__(spec, weights, rt)
+        self.size = int(spec["size"])
+        self.eps = float(spec["eps"])
+        if not self.eps > 0.0:
+            raise ValueError("LayerNorm needs a positive eps")
+        self.weight = rt.vector(weights["weight"])
+
+    def forward(self, ctx, x, out=None, rows=None):
+        count = x.shape[0] if rows is None else rows.numel()
+        if out is None:
+            out = self.rt.empty((count, self.size))
+        return self.rt.ops.layernorm(x, self.weight, self.eps, out, rows=rows)
+
+    def row_form(self):
+        return self.weight, self.eps, True
+
+
 register_part("norm", "rms", RMSNorm)
+register_part("norm", "layer", LayerNorm)
 register_part("norm", "rms_scalar", ScalarRMSNorm)

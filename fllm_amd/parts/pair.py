@@ -3,7 +3,8 @@
 `MixerPair` wraps two mixers (`left`, `right`: their PartSpecs; their tensors are listed under `left.<name>` and
 `right.<name>`).  Either may keep pages (at most one of them: a run entry has one place in a cache group) and either may
 keep state, which the pair names `left.<name>` / `right.<name>` beside each other.  Both must be able to store their output
-as a branch; the sum is taken in float32.
+as a branch; the sum is taken in float32.  `out_norm_eps`: each output passes an RMS norm over the model's width first, with the
+weights `left_out` and `right_out`.
 """
 from __future__ import annotations
 
@@ -12,7 +13,7 @@ from types import SimpleNamespace
 import torch
 
 from ..registry import part_class, register_part
-from .base import Mixer, StateNeed, fused_form
+from .base import INIT_NORM, Mixer, StateNeed, fused_form
 
 
 class MixerPair(Mixer):
@@ -20,7 +21,7 @@ class MixerPair(Mixer):
 
     @classmethod
     def tensor_shapes(cls, spec):
-        shapes = {}
+        shapes = {f"{side}_out": ((spec["size"],), INIT_NORM) for side in ("left", "right")} if spec.get("out_norm_eps") else {}
         for side in ("left", "right"):
             inner = spec[side]
             for name, shape in part_class("mixer", inner.kind).tensor_shapes(inner).items():
@@ -31,6 +32,8 @@ class MixerPair(Mixer):
         super().__init__(spec, weights, rt)
         self.size = int(spec["size"])
         self.scales = (float(spec.get("left_scale", 1.0)), float(spec.get("right_scale", 1.0)))
+        self.out_eps = float(spec.get("out_norm_eps") or 0.0)
+        self.out_weights = [rt.vector(weights[f"{side}_out"]) for side in ("left", "right")] if self.out_eps > 0.0 else None
         self.sides = []
         for side in ("left", "right"):
             inner = spec[side]
@@ -120,7 +123,10 @@ class MixerPair(Mixer):
 
     def _sum(self, outs, residual, branch) -> None:
         ops = self.rt.ops
-        if branch is not None:
+        if self.out_weights is not None:
+            ops.normed_pair_sum(branch if branch is not None else residual, outs[0], self.out_weights[0], self.scales[0], outs[1],
+                                self.out_weights[1], self.scales[1], self.out_eps, accumulate=branch is None)
+        elif branch is not None:
             ops.weighted_sum(branch, outs[0], self.scales[0], outs[1], self.scales[1])
         else:
             ops.weighted_sum(residual, outs[0], self.scales[0], outs[1], self.scales[1], accumulate=True)

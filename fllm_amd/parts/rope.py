@@ -8,7 +8,7 @@ phase = position * inv[l] in float32; cos and sin are evaluated in float64 and s
 cos and sin by a magnitude (rope.rs:70-110); `longrope` divides the frequencies by one of two lists of
 per-lane factors, the long one when the tables reach beyond the original context, and multiplies cos and sin
 by its attention factor (rope.rs:30-36, :58-61).  All of it in float32 up to the phase, as the reference.
-`precise` (plain and `yarn` tables): frequencies and phases are computed in float64 and only cos and sin are rounded to
+`precise` (plain, `llama3` and `yarn` tables): frequencies and phases are computed in float64 and only cos and sin are rounded to
 float32, for designs whose positions are checked more closely than a float32 product of position and frequency allows.
 """
 from __future__ import annotations
@@ -24,8 +24,9 @@ from .base import Part
 PAIR_HALF, PAIR_INTERLEAVED = 0, 1
 
 
-def llama3_divisors(dims: int, theta: float, factor: float, low: float, high: float, original: float):
-    """float64 per-lane divisors, returned as a float32 tensor [dims/2]."""
+def llama3_divisors(dims: int, theta: float, factor: float, low: float, high: float, original: float,
+                    kind: torch.dtype = torch.float32):
+    """float64 per-lane divisors, returned as a tensor [dims/2] of `kind`."""
     out = []
     low_wavelength = original / low
     high_wavelength = original / high
@@ -40,7 +41,7 @@ def llama3_divisors(dims: int, theta: float, factor: float, low: float, high: fl
             smooth = (original / wavelength - low) / (high - low)
             scale = 1.0 / ((1.0 - smooth) / factor + smooth)
         out.append(scale)
-    return torch.tensor(out, dtype=torch.float64).to(torch.float32)
+    return torch.tensor(out, dtype=torch.float64).to(kind)
 
 
 class Rotary(Part):
@@ -56,8 +57,8 @@ class Rotary(Part):
             raise ValueError("rotary dims must be even and positive")
         positions = int(min(rt.max_context, spec.get("max_position", rt.max_context)))
         self.precise = bool(spec.get("precise", False))
-        if self.precise and self.scaling not in ("none", "yarn"):
-            raise ValueError("precise tables are built for plain and yarn scaling")
+        if self.precise and self.scaling not in ("none", "yarn", "llama3"):
+            raise ValueError("precise tables are built for plain, llama3 and yarn scaling")
         key = ("rotary", self.dims, self.theta, self.scaling, positions, self.precise) + tuple(
             tuple(v) if isinstance(v, (list, tuple)) else v
             for v in (spec.get(k) for k in ("factor", "low_freq_factor", "high_freq_factor", "original_max_position",
@@ -82,7 +83,8 @@ class Rotary(Part):
         if self.scaling == "llama3":
             s = self.spec
             inv = inv / llama3_divisors(self.dims, self.theta, float(s["factor"]), float(s["low_freq_factor"]),
-                                        float(s["high_freq_factor"]), float(s["original_max_position"]))
+                                        float(s["high_freq_factor"]), float(s["original_max_position"]),
+                                        torch.float64 if self.precise else torch.float32)
         f32 = lambda v: torch.tensor(float(v), dtype=torch.float32)
         if self.scaling == "yarn":
             return self._build_yarn(positions, inv)

@@ -13,6 +13,7 @@ from typing import Dict, List, Tuple
 import torch
 
 from ..config.spec import ModelSpec, PartSpec
+from ..parts.base import SizeFromFile
 from ..registry import part_class
 from .safetensors_io import open_checkpoint
 
@@ -89,6 +90,10 @@ def canonical_names(spec: ModelSpec, names) -> Dict[str, str]:
     return out
 
 
+def _fits(got, want) -> bool:
+    return len(got) == len(want) and all(isinstance(w, SizeFromFile) or int(g) == int(w) for g, w in zip(got, want))
+
+
 def check_tensors(spec: ModelSpec, shapes: Dict[str, tuple]) -> None:
     """Raises `WeightsError` unless `shapes` (name -> shape of what a checkpoint holds) fits."""
     required, optional, _ = expected_tensors(spec)
@@ -98,7 +103,7 @@ def check_tensors(spec: ModelSpec, shapes: Dict[str, tuple]) -> None:
     wrong = []
     for n, got in shapes.items():
         want = required.get(n, optional.get(n))
-        if want is not None and tuple(got) != tuple(want):
+        if want is not None and not _fits(got, want):
             wrong.append((n, tuple(got), tuple(want)))
     if missing or unexpected or wrong:
         raise WeightsError(sorted(missing), sorted(unexpected), sorted(wrong))

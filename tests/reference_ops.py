@@ -472,10 +472,11 @@ class ReferenceOps:
             out[r, 2 * nq:] = qkv[r, 2 * nq:2 * nq + heads * vdim].to(out.dtype)
         return out
 
-    def group_norm_gate(self, x, eps, group, gate, out, activation="silu"):
+    def group_norm_gate(self, x, eps, group, gate, out, activation="silu", weight=None):
         rows, width = x.shape
         v = x.double().view(rows, width // group, group)
-        v = (v / torch.sqrt((v * v).mean(-1, keepdim=True) + eps)).view(rows, width)
+        v = v / torch.sqrt((v * v).mean(-1, keepdim=True) + eps)
+        v = (v if weight is None else v * weight.double()).view(rows, width)
         g = gate.double()
         g = g / (1.0 + torch.exp(-g)) if activation == "silu" else torch.sigmoid(g)
         out.copy_((v * g).to(out.dtype))
@@ -520,6 +521,158 @@ class ReferenceOps:
     def weighted_sum(self, out, x, a, y, b, accumulate=False):
         v = a * x.double() + b * y.double()
         out.copy_(((out.double() + v) if accumulate else v).to(out.dtype))
+        return out
+
+    # ---- layer norms; convolved attention whose mask keeps first tokens or whose heads' weights are mixed; recurrences with
+    # gates of their own; what a token brings beside the stream ----
+    def layernorm(self, x, weight, eps, out, rows=None):
+        src = (x if rows is None else x[rows.long()]).double()
+        d = src - src.mean(-1, keepdim=True)
+        out.copy_((d / torch.sqrt((d * d).mean(-1, keepdim=True) + eps) * weight.double()).to(out.dtype))
+        return out
+
+    def layernorm_pair(self, x, w1, eps1, out1, w2=None, eps2=None, out2=None):
+        self.layernorm(x, w1, eps1, out1)
+        if w2 is not None:
+            self.layernorm(x, w2, eps1 if eps2 is None else eps2, out2)
+        return out1, out2
+
+    def softcap_(self, x, cap):
+        x.copy_((cap * torch.tanh(x.double() / cap)).to(x.dtype))
+        return x
+
+    def cast_rows(self, x, out):
+        out.copy_(x.to(out.dtype))
+        return out
+
+    def gelu_side(self, z, ids, table, offset, out):
+        z = z.double()
+        e = table[ids.long(), offset:offset + z.shape[1]].double()
+        out.copy_((0.5 * z * (1.0 + torch.tanh(math.sqrt(2.0 / math.pi) * (z + 0.044715 * z ** 3))) * e).to(out.dtype))
+        return out
+
+    def normed_pair_sum(self, out, x, wx, a, y, wy, b, eps, accumulate=False):
+        n = lambda t, w: t.double() / torch.sqrt((t.double() ** 2).mean(-1, keepdim=True) + eps) * w.double()
+        v = a * n(x, wx) + b * n(y, wy)
+        out.copy_(((out.double() + v) if accumulate else v).to(out.dtype))
+        return out
+
+    def conv_qkv_store(self, joint, conv, bias, state, q_weight, k_weight, eps, q_out, row_pos, row_seg, seg_start, slots, tables, cos, sin,
+                       k_pages, v_pages, heads, kv_heads, k_dim, v_dim, rope_dims, pairing, page_size, key_chunk, single_rows=False):
+        channels, taps = conv.shape
+        keep = taps - 1
+        nq, nk = heads * k_dim, kv_heads * k_dim
+        half = rope_dims // 2
+        starts = [int(v) for v in seg_start]
+        for s in range(len(starts) - 1):
+            r0, r1 = starts[s], starts[s + 1]
+            if r1 <= r0 or int(row_seg[r0]) < 0:
+                continue
+            slot = int(slots[s])
+            old = state[slot] if keep else joint[:0, :channels]
+            seq = torch.cat([old, joint[r0:r1, :channels]])
+            for t in range(r1 - r0):
+                pos = int(row_pos[r0 + t])
+                u = seq[t:t + taps].double()
+                if bias is not None:
+                    u = u + bias.double()
+                before = max(0, keep - pos)                  # taps that reach before the sequence's first token
+                u[:before] = 0.0
+                y = (u * conv.double().T).sum(0)
+                q = y[:nq].view(heads, k_dim).clone()
+                k = y[nq:nq + nk].view(kv_heads, k_dim).clone() if k_pages is not None else None
+                for z, w in ((q, q_weight), (k, k_weight)):
+                    if z is None:
+                        continue
+                    if w is not None:
+                        z.copy_(z / torch.sqrt((z * z).mean(-1, keepdim=True) + eps) * w.double())
+                    if half:
+                        c, sn = cos[pos].double(), sin[pos].double()
+                        ia = torch.arange(half) * 2 if pairing else torch.arange(half)
+                        ib = ia + 1 if pairing else ia + half
+                        a, b = z[:, ia].clone(), z[:, ib].clone()
+                        z[:, ia], z[:, ib] = a * c - b * sn, b * c + a * sn
+                q_out[r0 + t] = q.reshape(-1).to(q_out.dtype)
+                if k_pages is not None:
+                    page, off = int(tables[s, pos // page_size]), pos % page_size
+                    k_pages[page, :, :, off, :] = k.view(kv_heads, k_dim // key_chunk, key_chunk).to(k_pages.dtype)
+                    v_pages[page, :, :, off] = y[nq + nk:].view(kv_heads, v_dim).to(v_pages.dtype)
+            if keep:
+                state[slot] = seq[-keep:].clone()
+        return q_out
+
+    def masked_attention(self, q, k_pages, v_pages, tables, row_pos, row_seg, seg_start, out, heads, kv_heads, k_dim, v_dim, page_size,
+                         scale, key_chunk, chunk=0, window=0, keep_first=0, softcap=0.0, zero_sink=False, spread=False, max_context=0):
+        group = heads // kv_heads
+        for r in range(q.shape[0]):
+            seg = int(row_seg[r])
+            if seg < 0:
+                out[r] = 0
+                continue
+            pos = int(row_pos[r])
+            lo = pos - pos % chunk if chunk else (max(0, pos - window + 1) if window else 0)
+            keys = torch.cat([torch.arange(0, min(keep_first, lo)), torch.arange(lo, pos + 1)])
+            pages, offs = tables[seg, (keys // page_size).long()].long(), (keys % page_size).long()
+            k = k_pages[pages, :, :, offs, :].double().reshape(len(keys), kv_heads, k_dim)
+            v = v_pages[pages, :, :, offs].double()
+            qr = q[r].double().view(heads, k_dim)
+            for h in range(heads):
+                s = (k[:, h // group, :] @ qr[h]) * scale
+                if softcap:
+                    s = softcap * torch.tanh(s / softcap)
+                if zero_sink:
+                    p = torch.softmax(torch.cat([s, torch.zeros(1, dtype=s.dtype)]), dim=0)[:-1]
+                else:
+                    p = torch.softmax(s, dim=0)
+                if spread:                     # this head's weights on the values of every key/value head
+                    n = kv_heads * v_dim
+                    out[r, h * n:(h + 1) * n] = torch.einsum("n,ngd->gd", p, v).reshape(-1).to(out.dtype)
+                else:
+                    out[r, h * v_dim:(h + 1) * v_dim] = (p @ v[:, h // group, :]).to(out.dtype)
+        return out
+
+    def mix_heads(self, spread, talk, out, heads, kv_heads, v_dim):
+        rows = spread.shape[0]
+        a = spread.double().view(rows, heads, kv_heads, v_dim)
+        group = heads // kv_heads
+        for h in range(heads):
+            out[:, h * v_dim:(h + 1) * v_dim] = torch.einsum("g,rgd->rd", talk[h].double(), a[:, :, h // group]).to(out.dtype)
+        return out
+
+    def gated_linear_attention(self, qkv, z, bias, tau, query_scale, state, row_seg, seg_start, slots, out, heads, dim, vdim, form="auto"):
+        starts = [int(v) for v in seg_start]
+        out.zero_()
+        nq = heads * dim
+        for s in range(len(starts) - 1):
+            r0, r1 = starts[s], starts[s + 1]
+            if r1 <= r0 or int(row_seg[r0]) < 0:
+                continue
+            S = state[int(slots[s])].double()
+            for r in range(r0, r1):
+                row = qkv[r].double()
+                q, k = row[:nq].view(heads, dim) * query_scale, row[nq:2 * nq].view(heads, dim)
+                v = row[2 * nq:2 * nq + heads * vdim].view(heads, vdim)
+                alpha = torch.sigmoid(z[r].double() + bias.double()).view(heads, dim) ** (1.0 / tau)
+                S = alpha.unsqueeze(2) * S + k.unsqueeze(2) * v.unsqueeze(1)
+                out[r] = torch.einsum("hdv,hd->hv", S, q).reshape(-1).to(out.dtype)
+            state[int(slots[s])] = S.to(state.dtype)
+        return out
+
+    def min_recurrence(self, zxg, bias, state, row_seg, seg_start, slots, out):
+        n = out.shape[1]
+        starts = [int(v) for v in seg_start]
+        out.zero_()
+        for s in range(len(starts) - 1):
+            r0, r1 = starts[s], starts[s + 1]
+            if r1 <= r0 or int(row_seg[r0]) < 0:
+                continue
+            S = state[int(slots[s])].double()
+            for r in range(r0, r1):
+                row = zxg[r].double()
+                z, u, g = torch.sigmoid(row[:n] + bias[:n].double()), row[n:2 * n] + bias[n:].double(), row[2 * n:]
+                S = (1.0 - z) * S + z * torch.where(u >= 0, u + 0.5, torch.sigmoid(u))
+                out[r] = (S * g * torch.sigmoid(g)).to(out.dtype)
+            state[int(slots[s])] = S.to(state.dtype)
         return out
 
     def carry_ids(self, ids, source, previous):
