@@ -407,8 +407,21 @@ int fllm_sigmoid_attention(const void *q, int q_stride, const void *k_pages, con
 int fllm_rotate_scale(const void *qkv, int ld, float *out, const int32_t *row_pos, const float *cos_table, const float *sin_table,
                       int table_positions, int rows, int heads, int dim, int vdim, int rope_dims, float key_scale, int dtype,
                       hipStream_t stream);
-// out = x / rms(x over each group of `group` lanes) * act(gate), act silu or sigmoid; x float32 or of `dtype`.
-int fllm_group_norm_gate(const void *x, int x_dtype, float eps, int group, const void *gate, int gate_ld, void *out, int rows, int width,
+// Softmax attention over the row's own chunk of `chunk` positions (window 0), or over its last `window` positions and the first
+// `keep_first` of the sequence (chunk 0; both 0: every position up to the row): score = q . k * scale, with softcap > 0 then
+// softcap * tanh(score / softcap); zero_sink: the denominator holds one more term exp(0) without a value.  spread 0: out of `dtype`
+// [rows, heads * v_dim]; spread 1: every head's weights meet the values of every key/value head, out float32 [rows, heads, kv_heads,
+// v_dim].  fllm_mix_heads: out_h = sum_g talk[h, g] * spread[g][h's key/value head] ([rows, heads * v_dim] of `dtype`), which is what
+// head h gets when the heads' WEIGHTS are mixed by talk (float32 [heads, heads]) before they meet the values.
+int fllm_masked_attention(const void *q, int q_stride, const void *k_pages, const void *v_pages, const int32_t *tables, int table_stride,
+                          const int32_t *row_pos, const int32_t *row_seg, const int32_t *seg_start, int num_segs, void *out, int rows,
+                          int heads, int kv_heads, int head_dim, int v_dim, int page_size, float scale, float softcap, int zero_sink,
+                          int chunk, int window, int keep_first, int spread, int key_chunk, int dtype, int max_context, hipStream_t stream);
+int fllm_mix_heads(const float *spread, const float *talk, void *out, int rows, int heads, int kv_heads, int v_dim, int dtype,
+                   hipStream_t stream);
+// out = x / rms(x over each group of `group` lanes) * weight * act(gate), act silu or sigmoid, weight float32 [group] or null (1);
+// x float32 or of `dtype`.
+int fllm_group_norm_gate(const void *x, int x_dtype, const float *weight, float eps, int group, const void *gate, int gate_ld, void *out, int rows, int width,
                          int silu, int dtype, hipStream_t stream);
 // out = a x + b y (accumulate: out += a x + b y), float32.
 int fllm_weighted_sum(float *out, const float *x, float a, const float *y, float b, size_t total, int accumulate, hipStream_t stream);
@@ -427,6 +440,54 @@ int fllm_experts_up(const void *h, int ldh, const int32_t *ids, int rows, int to
 int fllm_experts_grouped_ungated(const void *h, int ldh, const int32_t *ids, int rows, int top, const void *w_up, const void *w_down,
                                  int E, int inter, int K, int N, void *act, float *out, int32_t *work, float *planes,
                                  hipStream_t stream);
+
+// ---- layer norms and the small passes around them (layer_norms.hip) ----
+// out1[i] = (x[r] - mean) * rsqrt(mean (x[r] - mean)^2 + eps1) * w1, r = rows ? rows[i] : i, and with w2 the same with w2 and eps2 in out2.
+int fllm_layernorm(const float *x, const int32_t *rows, const float *w1, float eps1, void *out1, const float *w2, float eps2, void *out2,
+                   int count, int width, int out_dtype, hipStream_t stream);
+// out = a x / rms(x) wx + b y / rms(y) wy over rows of `width` (accumulate: out += ..), float32.
+int fllm_normed_pair_sum(float *out, const float *x, const float *wx, float a, const float *y, const float *wy, float b, float eps, int rows,
+                         int width, int accumulate, hipStream_t stream);
+// out = x in `dtype`.
+int fllm_cast_rows(const float *x, void *out, size_t total, int dtype, hipStream_t stream);
+// x = cap * tanh(x / cap), in place.
+int fllm_softcap(float *x, size_t total, float cap, hipStream_t stream);
+// out[r, c] = gelu_tanh(z[r, c]) * table[ids[r], offset + c], rows of `dim`; table [vocab, table_width] of `dtype`.
+int fllm_gelu_side(const void *z, const int32_t *ids, const void *table, int vocab, int table_width, int offset, void *out, int rows, int dim,
+                   int dtype, hipStream_t stream);
+
+// ---- projections behind a short convolution (conv_store.hip) ----
+// Rows [q | k | v | ..] of `ld` elements (store_kv 0: q alone passes the convolution).  Channel c of the row at position p: y = sum_j
+// conv[c][j] u(p - taps + 1 + j), u = the product + bias[c] (bias may be null), 0 before position 0; products before the step's first
+// row come from state[slots][taps - 1][channels] (of `dtype`, without the biases), which afterwards holds the sequence's last taps - 1.
+// Then, with q_weight and k_weight ([k_dim], float32; null: none) an RMS norm of every head of q and of k; rotary on the first
+// rope_dims lanes (pairing 0: i with i + rope_dims / 2; 1: 2i with 2i + 1); queries to q_out, keys and values into the pages.
+// single_rows: every segment has one row (the state moves on in the same kernel).
+int fllm_conv_qkv_store(const void *joint, int ld, const float *conv, int taps, const float *bias, void *state, const float *q_weight,
+                        const float *k_weight, float eps, void *q_out, const int32_t *row_pos, const int32_t *row_seg,
+                        const int32_t *seg_start, const int32_t *slots, int num_segs, const int32_t *tables, int table_stride,
+                        const float *cos_table, const float *sin_table, int table_positions, void *k_pages, void *v_pages, int rows,
+                        int heads, int kv_heads, int k_dim, int v_dim, int rope_dims, int pairing, int page_size, int key_chunk, int dtype,
+                        int store_kv, int single_rows, hipStream_t stream);
+
+// ---- recurrences whose gates the token chooses (gated_recurrences.hip, gated_linear_mfma.hip) ----
+// Per head S <- diag(alpha_t) S + k_t v_t^T, o_t = S^T (query_scale q_t), alpha = sigmoid(z + bias)^(1 / tau), one number a key channel:
+// z float32 [rows, heads * dim], bias float32 [heads * dim]; S float32 state[slots][heads][dim][vdim]; q, k (heads * dim) and v
+// (heads * vdim) columns of rows of `ld` elements; out float32 [rows, heads * vdim].  form 0: portions of prompts run chunks of 16
+// tokens on the matrix cores in float32 where the sizes allow (dim a multiple of 16 up to 128, vdim a multiple of 16), all else
+// token after token; 1: token after token; 2: chunks, an error where the sizes do not allow them.  `carried` (null, or
+// fllm_gated_linear_carried_floats floats): with it the chunked form cuts long segments into parts that run side by side.
+int fllm_gated_linear_attention(const void *q, const void *k, const void *v, int ld, const float *z, const float *bias, float tau,
+                                float query_scale, float *state, const int32_t *row_seg, const int32_t *seg_start, const int32_t *slots,
+                                int num_segs, float *out, int rows, int heads, int dim, int vdim, int form, int dtype, float *carried,
+                                hipStream_t stream);
+size_t fllm_gated_linear_carried_floats(int rows, int num_segs, int heads, int dim, int vdim);
+// S <- (1 - z) S + z c lane by lane over each segment's rows [a | x | g | ..] of `ld` elements: z = sigmoid(a + bias[0 ..]), u = x +
+// bias[width ..], c = u + 1/2 where u >= 0 and sigmoid(u) below; out = S * silu(g) of `dtype` [rows, width]; S float32
+// state[slots][width].  `carried`: fllm_min_recurrence_carried_floats floats (none needed where that is 0).
+int fllm_min_recurrence(const void *zxg, int ld, const float *bias, float *state, const int32_t *row_seg, const int32_t *seg_start,
+                        const int32_t *slots, int num_segs, void *out, int rows, int width, int dtype, float *carried, hipStream_t stream);
+size_t fllm_min_recurrence_carried_floats(int rows, int num_segs, int width);
 
 #ifdef __cplusplus
 }

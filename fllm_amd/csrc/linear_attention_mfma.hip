@@ -25,6 +25,7 @@
 // The powers a^0 .. a^32 come from the decay's float pair in double precision, once a workgroup.
 #include "api.h"
 #include "common.h"
+#include "segment_parts.h"
 
 namespace {
 
@@ -34,24 +35,6 @@ constexpr int kLDV = 48;          // row stride of V in LDS: lane groups 16 bank
 constexpr int kLDP = 33;
 constexpr int kThreads = 256;
 constexpr int kPart = 256;        // tokens a part, where a long segment is cut into parts that run side by side
-
-// Where part `part` of the segment that begins at row seg_r0 keeps its state among the carried ones: no two parts of a step
-// share an index, and the largest is below rows / kPart + segments.
-__host__ __device__ inline int carried_index(int seg_r0, int seg, int part) { return seg_r0 / kPart + seg + part; }
-
-// The grid of a step in parts has one workgroup (times heads and slices) an index that a part may have: workgroup w finds the
-// last segment whose first index is not above w (the first indices grow with the segment) and is that segment's part
-// w - first index, if the segment has so many.
-__device__ inline void find_part(int w, const int32_t *seg_start, int num_segs, int &seg, int &part) {
-    int lo = 0, hi = num_segs - 1;
-    while (lo < hi) {
-        const int mid = (lo + hi + 1) >> 1;
-        if (carried_index(seg_start[mid], mid, 0) <= w) lo = mid;
-        else hi = mid - 1;
-    }
-    seg = lo;
-    part = w - carried_index(seg_start[lo], lo, 0);
-}
 
 // silu of a projection: float32 rows get the library's exponential and a division; bfloat16 rows, whose own rounding is
 // 2^-9, the hardware's exponential and reciprocal (a few units in the last place of a float), a quarter of the instructions
@@ -86,7 +69,7 @@ linear_attention_chunked_kernel(const T *__restrict__ q, const T *__restrict__ k
     // in_parts: a segment is cut into parts of kPart tokens, a workgroup a part; every part but the first starts from
     // zeros, and every part of a segment of several leaves its state in `carried` for the kernel that follows
     int seg = blockIdx.x, part = 0;
-    if (in_parts) find_part(blockIdx.x, seg_start, num_segs, seg, part);
+    if (in_parts) find_part<kPart>(blockIdx.x, seg_start, num_segs, seg, part);
     const int h = blockIdx.y, j0 = blockIdx.z * kVB;
     const int seg_r0 = seg_start[seg], seg_n = seg_start[seg + 1] - seg_r0;
     if (part < 0 || seg_n <= part * kPart) return;
@@ -116,7 +99,7 @@ linear_attention_chunked_kernel(const T *__restrict__ q, const T *__restrict__ k
             for (int r = 0; r < 4; r++)
                 S[b][vj][r] = (part == 0 && di < key_blocks && col < vdim) ? mine[(size_t)(16 * di + 4 * g + r) * vdim + col] : 0.f;
         }
-    if (parts > 1) mine = carried + ((size_t)carried_index(seg_r0, seg, part) * heads + h) * dim * vdim;
+    if (parts > 1) mine = carried + ((size_t)part_index<kPart>(seg_r0, seg, part) * heads + h) * dim * vdim;
 
     // 1. the chunk's q, k, v: 16 bytes a load, all of a thread's loads in flight at once, and the next chunk's loads issued
     // before this chunk's products, so that a chunk waits for memory once at most
@@ -311,7 +294,7 @@ linear_attention_carry_kernel(const T *__restrict__ q, int ld, const float *__re
     float *Part = Qs + kC * LDQ;               // [wave][block][register][lane]
     float *pw = Part + 4 * 4 * 4 * 64;         // a^(c0 + 1) .. a^(c0 + kC)
     int seg, part;
-    find_part(blockIdx.x, seg_start, num_segs, seg, part);
+    find_part<kPart>(blockIdx.x, seg_start, num_segs, seg, part);
     const int h = blockIdx.y, j0 = blockIdx.z * kVB;
     const int seg_r0 = seg_start[seg], seg_n = seg_start[seg + 1] - seg_r0;
     if (part <= 0 || seg_n <= part * kPart || row_seg[seg_r0] < 0) return;
@@ -326,7 +309,7 @@ linear_attention_carry_kernel(const T *__restrict__ q, int ld, const float *__re
 
     f32x4_t S[NB][2];
     auto add_carried = [&](int i, float scale) {     // S = scale S + U_i
-        const float *u = carried + ((size_t)carried_index(seg_r0, seg, i) * heads + h) * dim * vdim;
+        const float *u = carried + ((size_t)part_index<kPart>(seg_r0, seg, i) * heads + h) * dim * vdim;
 #pragma unroll
         for (int b = 0; b < NB; b++)
 #pragma unroll

@@ -9,8 +9,13 @@
 //   pooled_window_attention  a row sees its last `window` tokens and one mean key and value for every block that lies wholly
 //                            before them; one softmax over both kinds.
 //   sigmoid_attention        no softmax: key j weighs sigmoid(cap * tanh(s / cap) - r1 ln(1 + r2 (pos - j)) + pb) on its own.
+//   masked_attention         softmax over the row's own chunk of positions, or over a window and the sequence's first tokens; scores
+//                            capped where asked, one more term of score 0 in the denominator where asked; a head's weights meet
+//                            the values of its own key/value head, or (spread) of every key/value head.
+//   mix_heads                out_h = sum_g talk[h][g] (head g's weights times the values of h's key/value head).
 //   rotate_scale             q and k of a linear attention rotated and k scaled, in float32, values beside them.
-//   group_norm_gate          every group of lanes divided by its root mean square, times silu or sigmoid of a gate.
+//   group_norm_gate          every group of lanes divided by its root mean square, times a weight a lane of a group where there is
+//                            one, times silu or sigmoid of a gate.
 //   weighted_sum, stream_concat, activation: the small passes around them.
 //
 // A row's result depends on its own position, pages and slot alone, never on the rest of the batch.
@@ -28,6 +33,12 @@ int fllm_sigmoid_attention_bf16_fast(const void *q, int q_stride, const void *k_
                                      int num_segs, void *out, int rows, int heads, int kv_heads, int head_dim, int v_dim, int page_size,
                                      float scale, float softcap, const float *r1, const float *r2, const float *pb, float temp_coef,
                                      int temp_every, int max_context, hipStream_t stream);
+
+int fllm_masked_attention_bf16_fast(const void *q, int q_stride, const void *k_pages, const void *v_pages, const int32_t *tables,
+                                    int table_stride, const int32_t *row_pos, const int32_t *row_seg, const int32_t *seg_start,
+                                    int num_segs, void *out, int rows, int heads, int kv_heads, int head_dim, int v_dim, int page_size,
+                                    float scale, float softcap, int zero_sink, int chunk, int window, int keep_first, int spread,
+                                    int max_context, hipStream_t stream);
 
 namespace {
 
@@ -408,6 +419,94 @@ sigmoid_attention_kernel(const T *__restrict__ q, int q_stride, const T *__restr
     }
 }
 
+// ---- softmax over a chunk, or over a window and the first tokens ---------------------------------------------------------------
+// grid (rows, heads, spread ? kv_heads : 1).  The row's keys in one line: the first tokens 0 .. nf - 1 that the window has passed,
+// then the positions lo .. pos.  O: T, or float with `spread` (out[row][head][value head][v_dim]).
+template <typename T, typename O>
+__global__ void __launch_bounds__(kBlock)
+masked_attention_kernel(const T *__restrict__ q, int q_stride, const T *__restrict__ k_pages, const T *__restrict__ v_pages,
+                        const int32_t *__restrict__ tables, int table_stride, const int32_t *__restrict__ row_pos,
+                        const int32_t *__restrict__ row_seg, O *__restrict__ out, int heads, int kv_heads, int head_dim, int v_dim,
+                        int page_size, float scale, float softcap, int zero_sink, int chunk, int window, int keep_first, int key_chunk,
+                        int vd_pad) {
+    extern __shared__ float smem[];
+    float *qs = smem;                                   // head_dim (rounded up to a multiple of 2)
+    float *sc = qs + ((head_dim + 1) & ~1);             // kBlock
+    float *scratch = sc + kBlock;                       // kWaves (+ padding to 8 bytes)
+    long long *voff = (long long *)(scratch + 2 * ((kWaves + 1) / 2));   // kBlock
+    int *vstep = (int *)(voff + kBlock);                // kBlock
+    float *buf = (float *)(vstep + kBlock);             // kMaxLanes * kBlock
+    const int r = blockIdx.x, h = blockIdx.y;
+    const int seg = row_seg[r];
+    O *dst = out + (((size_t)r * heads + h) * gridDim.z + blockIdx.z) * v_dim;
+    if (seg < 0) {
+        for (int c = threadIdx.x; c < v_dim; c += kBlock) dst[c] = from_f32<O>(0.f);
+        return;
+    }
+    const int pos = row_pos[r];
+    const int kvh = h / (heads / kv_heads), vh = gridDim.z > 1 ? (int)blockIdx.z : kvh;
+    int lo = window > 0 && pos - window + 1 > 0 ? pos - window + 1 : 0;
+    if (chunk > 0) lo = pos - pos % chunk;
+    const int nf = keep_first < lo ? keep_first : lo;
+    const int n = nf + (pos - lo + 1);
+    const int32_t *tbl = tables + (size_t)seg * table_stride;
+    const T *qrow = q + (size_t)r * q_stride + (size_t)h * head_dim;
+    for (int c = threadIdx.x; c < head_dim; c += kBlock) qs[c] = to_f32<T>(qrow[c]);
+    __syncthreads();
+    const size_t chunk_step = (size_t)page_size * key_chunk;
+    float m = zero_sink ? 0.f : -INFINITY, l = zero_sink ? 1.f : 0.f;      // the sink: a term exp(0) that is there from the start
+    float acc[kMaxLanes] = {0.f, 0.f};
+    for (int c0 = 0; c0 < n; c0 += kBlock) {
+        const int t = c0 + threadIdx.x;
+        float s = -INFINITY;
+        if (t < n) {
+            const int key = t < nf ? t : lo + (t - nf), page = tbl[key / page_size], off = key % page_size;
+            const T *kr = k_pages + key_at(page, kv_heads, kvh, page_size, head_dim, off, 0, key_chunk);
+            s = key_dot<T>(qs, kr, head_dim, chunk_step, key_chunk) * scale;
+            if (softcap > 0.f) s = softcap * tanhf(s / softcap);
+            voff[threadIdx.x] = (long long)(((size_t)page * kv_heads + vh) * v_dim * page_size + off);
+            vstep[threadIdx.x] = page_size;
+        }
+        const float m_new = fmaxf(m, block_max<kWaves>(s, scratch));
+        const float alpha = expf(m - m_new);
+        const float p = t < n ? expf(s - m_new) : 0.f;
+        sc[threadIdx.x] = p;
+        l = l * alpha + block_sum<kWaves>(p, scratch);   // the barriers inside also publish sc[], voff[] and vstep[]
+        const int count = n - c0 < kBlock ? n - c0 : kBlock;
+#pragma unroll
+        for (int i = 0; i < kMaxLanes; i++) acc[i] *= alpha;
+        add_values<T, false>(acc, sc, voff, vstep, count, v_pages, nullptr, v_dim, vd_pad);
+        m = m_new;
+        __syncthreads();
+    }
+    merge_groups(acc, buf, vd_pad);
+    const float inv = 1.0f / l;
+    if (threadIdx.x < vd_pad) {
+#pragma unroll
+        for (int i = 0; i < kMaxLanes; i++) {
+            const int c = threadIdx.x + i * vd_pad;
+            if (c < v_dim) dst[c] = from_f32<O>(acc[i] * inv);
+        }
+    }
+}
+
+// spread [row][head][value head][v_dim] float32 -> out[row][head][v_dim]: out_h = sum_g talk[h][g] spread[g][value head of h].
+// grid (rows, blocks of outputs); the sum runs in head order.
+template <typename T>
+__global__ void __launch_bounds__(kBlock)
+mix_heads_kernel(const float *__restrict__ spread, const float *__restrict__ talk, T *__restrict__ out, int heads, int kv_heads, int v_dim) {
+    const size_t r = blockIdx.x;
+    const int o = blockIdx.y * kBlock + threadIdx.x;
+    if (o >= heads * v_dim) return;
+    const int h = o / v_dim, c = o - h * v_dim, vh = h / (heads / kv_heads);
+    const float *src = spread + (r * heads * kv_heads + vh) * v_dim + c;
+    const float *tk = talk + (size_t)h * heads;
+    float acc = 0.f;
+#pragma unroll 8
+    for (int g = 0; g < heads; g++) acc = fmaf(tk[g], src[(size_t)g * kv_heads * v_dim], acc);
+    out[r * heads * v_dim + o] = from_f32<T>(acc);
+}
+
 // ---- operands of a linear attention: rotated, scaled, float32 ----------------------------------------------------------------
 template <typename T>
 __global__ void __launch_bounds__(kBlock)
@@ -437,8 +536,8 @@ rotate_scale_kernel(const T *__restrict__ qkv, int ld, float *__restrict__ out, 
 // ---- a norm a group of lanes, gated -----------------------------------------------------------------------------------------
 template <typename X, typename T>
 __global__ void __launch_bounds__(kBlock)
-group_norm_gate_kernel(const X *__restrict__ x, float eps, int group, const T *__restrict__ gate, int gate_ld, T *__restrict__ out,
-                       int width, int silu) {
+group_norm_gate_kernel(const X *__restrict__ x, const float *__restrict__ weight, float eps, int group, const T *__restrict__ gate, int gate_ld,
+                       T *__restrict__ out, int width, int silu) {
     const size_t r = blockIdx.x;
     const int lane = threadIdx.x & (kWave - 1), wave = threadIdx.x / kWave;
     for (int g = wave; g < width / group; g += kWaves) {
@@ -450,7 +549,7 @@ group_norm_gate_kernel(const X *__restrict__ x, float eps, int group, const T *_
         for (int c = lane; c < group; c += kWave) {
             const float z = to_f32<T>(gate[r * gate_ld + (size_t)g * group + c]);
             const float sg = 1.0f / (1.0f + expf(-z));
-            out[r * width + (size_t)g * group + c] = from_f32<T>(to_f32<X>(src[c]) * inv * (silu ? z * sg : sg));
+            out[r * width + (size_t)g * group + c] = from_f32<T>(to_f32<X>(src[c]) * inv * (weight != nullptr ? weight[c] : 1.0f) * (silu ? z * sg : sg));
         }
     }
 }
@@ -637,6 +736,54 @@ extern "C" int fllm_sigmoid_attention(const void *q, int q_stride, const void *k
     return fllm_check_launch("sigmoid_attention");
 }
 
+extern "C" int fllm_masked_attention(const void *q, int q_stride, const void *k_pages, const void *v_pages, const int32_t *tables, int table_stride,
+                                     const int32_t *row_pos, const int32_t *row_seg, const int32_t *seg_start, int num_segs, void *out,
+                                     int rows, int heads, int kv_heads, int head_dim, int v_dim, int page_size, float scale, float softcap,
+                                     int zero_sink, int chunk, int window, int keep_first, int spread, int key_chunk, int dtype,
+                                     int max_context, hipStream_t stream) {
+    FLLM_REQUIRE(rows >= 0 && heads > 0 && heads <= 65535 && kv_heads > 0 && kv_heads <= 65535 && head_dim > 0 && v_dim > 0 && page_size > 0 &&
+                     table_stride > 0, "masked_attention: bad sizes");
+    FLLM_REQUIRE(softcap >= 0.f && chunk >= 0 && window >= 0 && keep_first >= 0 && (chunk == 0 || window == 0) && (keep_first == 0 || window > 0),
+                 "masked_attention: a row sees its chunk, or a window with first tokens kept (chunk %d, window %d, first %d)", chunk, window, keep_first);
+    FLLM_REQUIRE(heads % kv_heads == 0, "masked_attention: %d heads are not a multiple of %d key/value heads", heads, kv_heads);
+    FLLM_REQUIRE(key_chunk > 0 && head_dim % key_chunk == 0, "masked_attention: keys of %d lanes in chunks of %d", head_dim, key_chunk);
+    FLLM_REQUIRE(v_dim <= kBlock * kMaxLanes, "masked_attention: values of %d lanes a head are more than %d", v_dim, kBlock * kMaxLanes);
+    FLLM_REQUIRE(q_stride >= heads * head_dim, "masked_attention: q_stride %d is shorter than heads * head_dim", q_stride);
+    FLLM_REQUIRE(q && k_pages && v_pages && tables && row_pos && row_seg && out, "masked_attention: operands missing");
+    if (rows == 0) return 0;
+    if (dtype == FLLM_BF16 && key_chunk == 8) {
+        const int fast = fllm_masked_attention_bf16_fast(q, q_stride, k_pages, v_pages, tables, table_stride, row_pos, row_seg, seg_start,
+                                                         num_segs, out, rows, heads, kv_heads, head_dim, v_dim, page_size, scale, softcap,
+                                                         zero_sink, chunk, window, keep_first, spread, max_context, stream);
+        if (fast <= 0) return fast;
+    }
+    const int vd_pad = pow2_lanes(v_dim);
+    const size_t smem = (size_t)(((head_dim + 1) & ~1) + kBlock + 2 * ((kWaves + 1) / 2)) * sizeof(float) + (size_t)kBlock * (sizeof(long long) + sizeof(int)) +
+                        (size_t)kMaxLanes * kBlock * sizeof(float);
+    FLLM_REQUIRE(smem <= 64 * 1024, "masked_attention: heads of %d lanes do not fit into LDS", head_dim);
+    const dim3 grid(rows, heads, spread ? kv_heads : 1);
+#define FLLM_MASKED(T, O)                                                                                                                  hipLaunchKernelGGL((masked_attention_kernel<T, O>), grid, dim3(kBlock), smem, stream, (const T *)q, q_stride, (const T *)k_pages,                          (const T *)v_pages, tables, table_stride, row_pos, row_seg, (O *)out, heads, kv_heads, head_dim, v_dim, page_size,                        scale, softcap, zero_sink, chunk, window, keep_first, key_chunk, vd_pad)
+    if (dtype == FLLM_F32) FLLM_MASKED(float, float);
+    else if (dtype == FLLM_BF16 && spread) FLLM_MASKED(bf16_t, float);
+    else if (dtype == FLLM_BF16) FLLM_MASKED(bf16_t, bf16_t);
+    else FLLM_REQUIRE(false, "masked_attention: unknown dtype %d", dtype);
+#undef FLLM_MASKED
+    return fllm_check_launch("masked_attention");
+}
+
+extern "C" int fllm_mix_heads(const float *spread, const float *talk, void *out, int rows, int heads, int kv_heads, int v_dim, int dtype,
+                              hipStream_t stream) {
+    FLLM_REQUIRE(rows >= 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && v_dim > 0, "mix_heads: bad sizes");
+    FLLM_REQUIRE(spread && talk && out, "mix_heads: operands missing");
+    if (rows == 0) return 0;
+    const dim3 grid(rows, (heads * v_dim + kBlock - 1) / kBlock);
+    FLLM_REQUIRE(grid.y <= 65535, "mix_heads: too many heads");
+    if (dtype == FLLM_F32) hipLaunchKernelGGL(mix_heads_kernel<float>, grid, dim3(kBlock), 0, stream, spread, talk, (float *)out, heads, kv_heads, v_dim);
+    else if (dtype == FLLM_BF16) hipLaunchKernelGGL(mix_heads_kernel<bf16_t>, grid, dim3(kBlock), 0, stream, spread, talk, (bf16_t *)out, heads, kv_heads, v_dim);
+    else FLLM_REQUIRE(false, "mix_heads: unknown dtype %d", dtype);
+    return fllm_check_launch("mix_heads");
+}
+
 extern "C" int fllm_rotate_scale(const void *qkv, int ld, float *out, const int32_t *row_pos, const float *cos_table,
                                  const float *sin_table, int table_positions, int rows, int heads, int dim, int vdim, int rope_dims,
                                  float key_scale, int dtype, hipStream_t stream) {
@@ -656,12 +803,12 @@ extern "C" int fllm_rotate_scale(const void *qkv, int ld, float *out, const int3
     return fllm_check_launch("rotate_scale");
 }
 
-extern "C" int fllm_group_norm_gate(const void *x, int x_dtype, float eps, int group, const void *gate, int gate_ld, void *out, int rows,
+extern "C" int fllm_group_norm_gate(const void *x, int x_dtype, const float *weight, float eps, int group, const void *gate, int gate_ld, void *out, int rows,
                                     int width, int silu, int dtype, hipStream_t stream) {
     FLLM_REQUIRE(rows >= 0 && width > 0 && group > 0 && width % group == 0 && gate_ld >= width && eps > 0.f, "group_norm_gate: bad sizes");
     FLLM_REQUIRE(x && gate && out, "group_norm_gate: operands missing");
     if (rows == 0) return 0;
-#define FLLM_GROUPED(X, T) hipLaunchKernelGGL((group_norm_gate_kernel<X, T>), dim3(rows), dim3(kBlock), 0, stream, (const X *)x, eps, group, \
+#define FLLM_GROUPED(X, T) hipLaunchKernelGGL((group_norm_gate_kernel<X, T>), dim3(rows), dim3(kBlock), 0, stream, (const X *)x, weight, eps, group, \
                                               (const T *)gate, gate_ld, (T *)out, width, silu)
     if (x_dtype == FLLM_F32 && dtype == FLLM_F32) FLLM_GROUPED(float, float);
     else if (x_dtype == FLLM_F32 && dtype == FLLM_BF16) FLLM_GROUPED(float, bf16_t);

@@ -49,7 +49,7 @@ assert SAMPLE_ROW_BYTES == 32
 _lib = None
 
 
-ABI_VERSION = 17
+ABI_VERSION = 18
 
 
 def load_library(build_if_missing: bool = True):
@@ -147,7 +147,21 @@ def load_library(build_if_missing: bool = True):
                                    c_int, c_void],
         "fllm_rotate_scale": [c_void, c_int, c_void, c_void, c_void, c_void, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int,
                               c_void],
-        "fllm_group_norm_gate": [c_void, c_int, c_float, c_int, c_void, c_int, c_void, c_int, c_int, c_int, c_int, c_void],
+        "fllm_group_norm_gate": [c_void, c_int, c_void, c_float, c_int, c_void, c_int, c_void, c_int, c_int, c_int, c_int, c_void],
+        "fllm_layernorm": [c_void, c_void, c_void, c_float, c_void, c_void, c_float, c_void, c_int, c_int, c_int, c_void],
+        "fllm_normed_pair_sum": [c_void, c_void, c_void, c_float, c_void, c_void, c_float, c_float, c_int, c_int, c_int, c_void],
+        "fllm_cast_rows": [c_void, c_void, c_size, c_int, c_void],
+        "fllm_softcap": [c_void, c_size, c_float, c_void],
+        "fllm_gelu_side": [c_void, c_void, c_void, c_int, c_int, c_int, c_void, c_int, c_int, c_int, c_void],
+        "fllm_conv_qkv_store": [c_void, c_int, c_void, c_int, c_void, c_void, c_void, c_void, c_float, c_void, c_void, c_void, c_void, c_void,
+                                c_int, c_void, c_int, c_void, c_void, c_int, c_void, c_void, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
+                                c_int, c_int, c_int, c_int, c_int, c_void],
+        "fllm_masked_attention": [c_void, c_int, c_void, c_void, c_void, c_int, c_void, c_void, c_void, c_int, c_void, c_int, c_int, c_int,
+                                  c_int, c_int, c_int, c_float, c_float, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void],
+        "fllm_mix_heads": [c_void, c_void, c_void, c_int, c_int, c_int, c_int, c_int, c_void],
+        "fllm_gated_linear_attention": [c_void, c_void, c_void, c_int, c_void, c_void, c_float, c_float, c_void, c_void, c_void, c_void, c_int,
+                                        c_void, c_int, c_int, c_int, c_int, c_int, c_int, c_void, c_void],
+        "fllm_min_recurrence": [c_void, c_int, c_void, c_void, c_void, c_void, c_void, c_int, c_void, c_int, c_int, c_int, c_void, c_void],
         "fllm_weighted_sum": [c_void, c_void, c_float, c_void, c_float, c_size, c_int, c_void],
         "fllm_stream_concat": [c_void, c_void, c_void, c_int, c_float, c_void, c_int, c_int, c_int, c_void],
         "fllm_relu_squared": [c_void, c_void, c_size, c_int, c_void],
@@ -185,6 +199,10 @@ def load_library(build_if_missing: bool = True):
     lib.fllm_experts_grouped_plane_floats.restype = c_size
     lib.fllm_linear_attention_carried_floats.argtypes = [c_int, c_int, c_int, c_int, c_int]
     lib.fllm_linear_attention_carried_floats.restype = c_size
+    lib.fllm_gated_linear_carried_floats.argtypes = [c_int, c_int, c_int, c_int, c_int]
+    lib.fllm_gated_linear_carried_floats.restype = c_size
+    lib.fllm_min_recurrence_carried_floats.argtypes = [c_int, c_int, c_int]
+    lib.fllm_min_recurrence_carried_floats.restype = c_size
     lib.fllm_experts_grouped_work_ints.argtypes = [c_int, c_int]
     lib.fllm_experts_grouped_work_ints.restype = c_size
     lib.fllm_attention_workspace_bytes.argtypes = [c_int, c_int, c_int, c_int, c_int]
@@ -1283,9 +1301,9 @@ class Ops:
         return out
 
     def group_norm_gate(self, x: torch.Tensor, eps: float, group: int, gate: torch.Tensor, out: torch.Tensor,
-                        activation: str = "silu") -> torch.Tensor:
-        """out = x / sqrt(mean over each group of `group` lanes of x^2 + eps) * act(gate), act "silu" or "sigmoid"; `gate` may be a
-        column slice of a wider matrix."""
+                        activation: str = "silu", weight: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """out = x / sqrt(mean over each group of `group` lanes of x^2 + eps) * weight * act(gate), act "silu" or "sigmoid", `weight`
+        (float32 [group], None: 1) shared by the groups; `gate` may be a column slice of a wider matrix."""
         rows, width = x.shape
         _dense(x, "x")
         _need(activation in ("silu", "sigmoid"), f"activation {activation!r} unknown")
@@ -1294,7 +1312,9 @@ class Ops:
               "gate must be [rows, width] of out's type with unit column stride")
         _dense(out, "out", None, (rows, width))
         _need(out.dtype in _DTYPE_CODE and (x.dtype == torch.float32 or x.dtype == out.dtype), "group_norm_gate: x is float32 or of out's type")
-        self._check(self.lib.fllm_group_norm_gate(_ptr(x), _DTYPE_CODE[x.dtype], float(eps), int(group), _ptr(gate),
+        if weight is not None:
+            _dense(weight, "weight", torch.float32, (group,))
+        self._check(self.lib.fllm_group_norm_gate(_ptr(x), _DTYPE_CODE[x.dtype], _ptr(weight), float(eps), int(group), _ptr(gate),
                                                   gate.stride(0) if rows > 1 else width, _ptr(out), rows, width,
                                                   1 if activation == "silu" else 0, _DTYPE_CODE[out.dtype], self._stream()))
         return out
@@ -1388,6 +1408,217 @@ class Ops:
             return False
         self._check(code)
         return True
+
+    # ---- layer norms, convolved projections, masked attention, recurrences whose gates the token chooses --------------------
+    def layernorm(self, x: torch.Tensor, weight: torch.Tensor, eps: float, out: torch.Tensor, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """out = (x - mean) / sqrt(mean((x - mean)^2) + eps) * weight over float32 rows (`rows` selects some), out of either type."""
+        width = x.shape[-1]
+        _dense(x, "x", torch.float32)
+        _dense(weight, "weight", torch.float32, (width,))
+        count = x.shape[0] if rows is None else rows.numel()
+        if rows is not None:
+            _dense(rows, "rows", torch.int32)
+        _dense(out, "out", None, (count, width))
+        _need(out.dtype in _DTYPE_CODE, f"out dtype {out.dtype} unsupported")
+        self._check(self.lib.fllm_layernorm(_ptr(x), _ptr(rows), _ptr(weight), float(eps), _ptr(out), None, 0.0, None, count, width,
+                                            _DTYPE_CODE[out.dtype], self._stream()))
+        return out
+
+    def layernorm_pair(self, x: torch.Tensor, w1: torch.Tensor, eps1: float, out1: torch.Tensor,
+                       w2: Optional[torch.Tensor] = None, eps2: Optional[float] = None, out2: Optional[torch.Tensor] = None):
+        """Two layer norms of the same float32 rows in one pass over them (w2 and out2 None: one)."""
+        rows, width = x.shape
+        _dense(x, "x", torch.float32)
+        _dense(w1, "w1", torch.float32, (width,))
+        _dense(out1, "out1", None, (rows, width))
+        _need(out1.dtype in _DTYPE_CODE, f"out dtype {out1.dtype} unsupported")
+        _need((w2 is None) == (out2 is None), "the second norm needs a weight and an output")
+        if w2 is not None:
+            _dense(w2, "w2", torch.float32, (width,))
+            _dense(out2, "out2", out1.dtype, (rows, width))
+        self._check(self.lib.fllm_layernorm(_ptr(x), None, _ptr(w1), float(eps1), _ptr(out1), _ptr(w2), float(eps1 if eps2 is None else eps2),
+                                            _ptr(out2), rows, width, _DTYPE_CODE[out1.dtype], self._stream()))
+        return out1, out2
+
+    def normed_pair_sum(self, out: torch.Tensor, x: torch.Tensor, wx: torch.Tensor, a: float, y: torch.Tensor, wy: torch.Tensor, b: float,
+                        eps: float, accumulate: bool = False) -> torch.Tensor:
+        """out = a * x / rms(x) * wx + b * y / rms(y) * wy over rows (eps inside the root; `accumulate`: out += ..), float32."""
+        rows, width = out.shape
+        _dense(out, "out", torch.float32)
+        for name, t in (("x", x), ("y", y)):
+            _dense(t, name, torch.float32, (rows, width))
+        for name, t in (("wx", wx), ("wy", wy)):
+            _dense(t, name, torch.float32, (width,))
+        self._check(self.lib.fllm_normed_pair_sum(_ptr(out), _ptr(x), _ptr(wx), float(a), _ptr(y), _ptr(wy), float(b), float(eps), rows, width,
+                                                  1 if accumulate else 0, self._stream()))
+        return out
+
+    def cast_rows(self, x: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+        """out = the float32 rows x in out's type."""
+        _dense(x, "x", torch.float32)
+        _dense(out, "out", None, tuple(x.shape))
+        _need(out.dtype in _DTYPE_CODE, f"out dtype {out.dtype} unsupported")
+        self._check(self.lib.fllm_cast_rows(_ptr(x), _ptr(out), x.numel(), _DTYPE_CODE[out.dtype], self._stream()))
+        return out
+
+    def softcap_(self, x: torch.Tensor, cap: float) -> torch.Tensor:
+        """x = cap * tanh(x / cap), float32, in place."""
+        _dense(x, "x", torch.float32)
+        _need(cap > 0, "a cap must be positive")
+        self._check(self.lib.fllm_softcap(_ptr(x), x.numel(), float(cap), self._stream()))
+        return x
+
+    def gelu_side(self, z: torch.Tensor, ids: torch.Tensor, table: torch.Tensor, offset: int, out: torch.Tensor) -> torch.Tensor:
+        """out[r] = gelu_tanh(z[r]) * table[ids[r], offset : offset + dim]."""
+        rows, dim = z.shape
+        _dense(z, "z")
+        _need(z.dtype in _DTYPE_CODE, f"dtype {z.dtype} unsupported")
+        _dense(ids, "ids", torch.int32, (rows,))
+        _dense(table, "table", z.dtype)
+        _need(table.dim() == 2 and 0 <= offset and offset + dim <= table.shape[1], "the table's rows are too short")
+        _dense(out, "out", z.dtype, (rows, dim))
+        self._check(self.lib.fllm_gelu_side(_ptr(z), _ptr(ids), _ptr(table), table.shape[0], table.shape[1], int(offset), _ptr(out), rows, dim,
+                                            _DTYPE_CODE[z.dtype], self._stream()))
+        return out
+
+    def conv_qkv_store(self, joint: torch.Tensor, conv: torch.Tensor, bias: Optional[torch.Tensor], state: Optional[torch.Tensor],
+                       q_weight: Optional[torch.Tensor], k_weight: Optional[torch.Tensor], eps: float, q_out: torch.Tensor,
+                       row_pos: torch.Tensor, row_seg: torch.Tensor, seg_start: torch.Tensor, slots: torch.Tensor, tables: torch.Tensor,
+                       cos: torch.Tensor, sin: torch.Tensor, k_pages: Optional[torch.Tensor], v_pages: Optional[torch.Tensor], heads: int,
+                       kv_heads: int, k_dim: int, v_dim: int, rope_dims: int, pairing: int, page_size: int, key_chunk: int,
+                       single_rows: bool = False) -> torch.Tensor:
+        """Rows of a joint product [q | k | v | ..] (pages None: q alone): every channel convolved over time, y_t = sum_j conv[:, j] u_(t -
+        taps + 1 + j) with u the product + `bias`, 0 before position 0, the products before the step's first row from `state` [slots,
+        taps - 1, channels] (of joint's type), which then takes the sequence's last taps - 1; an RMS norm of every head of q and of k
+        with weights [k_dim] (None: none); rotary on the first `rope_dims` lanes (pairing 0: i with i + rope_dims / 2, 1: 2i with
+        2i + 1); queries to `q_out`, keys and values into the pages.  `single_rows`: every segment has one row."""
+        rows = joint.shape[0]
+        store = k_pages is not None
+        channels = heads * k_dim + (kv_heads * (k_dim + v_dim) if store else 0)
+        taps = conv.shape[1]
+        _need(joint.is_cuda and joint.dim() == 2 and joint.is_contiguous() and joint.dtype in _DTYPE_CODE, "joint must be dense rows on the GPU")
+        _need(joint.shape[1] >= channels, "joint rows are too short")
+        _dense(conv, "conv", torch.float32, (channels, taps))
+        if bias is not None:
+            _dense(bias, "bias", torch.float32, (channels,))
+        if q_weight is not None:
+            _dense(q_weight, "q_weight", torch.float32, (k_dim,))
+            _need(not store or k_weight is not None, "keys that are stored are normed too")
+            if k_weight is not None:
+                _dense(k_weight, "k_weight", torch.float32, (k_dim,))
+        _dense(q_out, "q_out", joint.dtype, (rows, heads * k_dim))
+        _dense(row_pos, "row_pos", torch.int32, (rows,))
+        _dense(row_seg, "row_seg", torch.int32, (rows,))
+        _dense(seg_start, "seg_start", torch.int32)
+        _dense(slots, "slots", torch.int32)
+        _dense(tables, "tables", torch.int32)
+        num_segs = seg_start.numel() - 1
+        _need(num_segs >= 1 and slots.numel() >= num_segs and tables.dim() == 2 and tables.shape[0] >= num_segs, "a slot and a table row a segment")
+        if taps > 1:
+            _need(state is not None, "the taps before a step need a state")
+            _dense(state, "state", joint.dtype, (state.shape[0], taps - 1, channels))
+        _dense(cos, "cos", torch.float32)
+        _dense(sin, "sin", torch.float32, tuple(cos.shape))
+        _need(cos.dim() == 2 and cos.shape[1] == rope_dims // 2, f"rotary tables must be [positions, {rope_dims // 2}]")
+        if store:
+            self._talking_pages(k_pages, v_pages, joint.dtype, kv_heads, k_dim, v_dim, page_size, key_chunk)
+        self._check(self.lib.fllm_conv_qkv_store(
+            _ptr(joint), joint.shape[1], _ptr(conv), taps, _ptr(bias), _ptr(state), _ptr(q_weight), _ptr(k_weight), float(eps), _ptr(q_out),
+            _ptr(row_pos), _ptr(row_seg), _ptr(seg_start), _ptr(slots), num_segs, _ptr(tables), tables.shape[1], _ptr(cos), _ptr(sin),
+            cos.shape[0], _ptr(k_pages), _ptr(v_pages), rows, heads, kv_heads, k_dim, v_dim, rope_dims, int(pairing), page_size, key_chunk,
+            _DTYPE_CODE[joint.dtype], 1 if store else 0, 1 if single_rows and rows == num_segs else 0, self._stream()))
+        return q_out
+
+    def masked_attention(self, q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, tables: torch.Tensor, row_pos: torch.Tensor,
+                         row_seg: torch.Tensor, seg_start: torch.Tensor, out: torch.Tensor, heads: int, kv_heads: int, k_dim: int, v_dim: int,
+                         page_size: int, scale: float, key_chunk: int, chunk: int = 0, window: int = 0, keep_first: int = 0,
+                         softcap: float = 0.0, zero_sink: bool = False, spread: bool = False, max_context: int = 0) -> torch.Tensor:
+        """Softmax attention over the row's own chunk of `chunk` positions, or over its last `window` positions and the first
+        `keep_first` of the sequence (both 0: everything up to the row); `softcap` > 0: softcap * tanh(score / softcap);
+        `zero_sink`: one more term exp(0) in the denominator.  `spread`: a head's weights meet the values of every key/value head,
+        out float32 [rows, heads * kv_heads * v_dim] (for `mix_heads`)."""
+        rows = q.shape[0]
+        _need(q.is_cuda and q.dim() == 2 and q.stride(1) == 1 and q.shape[1] == heads * k_dim and q.dtype in _DTYPE_CODE,
+              f"q must be [rows, {heads * k_dim}] of float32 or bfloat16 with unit column stride")
+        _need(heads % kv_heads == 0, f"{heads} heads are not a multiple of {kv_heads} key/value heads")
+        self._talking_pages(k_pages, v_pages, q.dtype, kv_heads, k_dim, v_dim, page_size, key_chunk)
+        _dense(tables, "tables", torch.int32)
+        _need(tables.dim() == 2, "tables must be [segments, pages]")
+        _dense(row_pos, "row_pos", torch.int32, (rows,))
+        _dense(row_seg, "row_seg", torch.int32, (rows,))
+        _dense(out, "out", *((torch.float32, (rows, heads * kv_heads * v_dim)) if spread else (q.dtype, (rows, heads * v_dim))))
+        self._segments(seg_start, tables, rows)
+        self._check(self.lib.fllm_masked_attention(
+            _ptr(q), q.stride(0) if rows > 1 else heads * k_dim, _ptr(k_pages), _ptr(v_pages), _ptr(tables), tables.shape[1], _ptr(row_pos),
+            _ptr(row_seg), _ptr(seg_start), seg_start.numel() - 1, _ptr(out), rows, heads, kv_heads, k_dim, v_dim, page_size, float(scale),
+            float(softcap), 1 if zero_sink else 0, int(chunk), int(window), int(keep_first), 1 if spread else 0, key_chunk,
+            _DTYPE_CODE[q.dtype], int(max_context), self._stream()))
+        return out
+
+    def mix_heads(self, spread: torch.Tensor, talk: torch.Tensor, out: torch.Tensor, heads: int, kv_heads: int, v_dim: int) -> torch.Tensor:
+        """out_h = sum_g talk[h, g] * spread[g][h's key/value head]; spread float32 [rows, heads * kv_heads * v_dim]."""
+        rows = out.shape[0]
+        _dense(spread, "spread", torch.float32, (rows, heads * kv_heads * v_dim))
+        _dense(talk, "talk", torch.float32, (heads, heads))
+        _dense(out, "out", None, (rows, heads * v_dim))
+        _need(out.dtype in _DTYPE_CODE, f"out dtype {out.dtype} unsupported")
+        self._check(self.lib.fllm_mix_heads(_ptr(spread), _ptr(talk), _ptr(out), rows, heads, kv_heads, v_dim, _DTYPE_CODE[out.dtype],
+                                            self._stream()))
+        return out
+
+    def gated_linear_attention(self, qkv: torch.Tensor, z: torch.Tensor, bias: torch.Tensor, tau: float, query_scale: float,
+                               state: torch.Tensor, row_seg: torch.Tensor, seg_start: torch.Tensor, slots: torch.Tensor, out: torch.Tensor,
+                               heads: int, dim: int, vdim: int, form: str = "auto") -> torch.Tensor:
+        """Per head S <- diag(alpha) S + k v^T, o = S^T (query_scale q), alpha = sigmoid(z + bias)^(1 / tau) (z float32 [rows, heads *
+        dim]); rows of `qkv` hold [q | k | v | ..]; S float32 state[slots, heads, dim, vdim]; out float32 [rows, heads * vdim].
+        `form`: "tokens" runs token after token, "chunks" 16 tokens at a time on the matrix cores in float32 (dim a multiple of 16 up
+        to 128, vdim a multiple of 16), "auto" chunks where a step holds portions of prompts and the sizes allow."""
+        rows = qkv.shape[0]
+        _need(qkv.is_cuda and qkv.dim() == 2 and qkv.stride(1) == 1 and qkv.dtype in _DTYPE_CODE, "qkv must be a row-major GPU matrix")
+        ld = qkv.stride(0) if rows > 1 else qkv.shape[1]
+        _need(qkv.shape[1] >= heads * (2 * dim + vdim), "qkv rows are too short")
+        _need(form in ("auto", "tokens", "chunks"), f"form {form!r} unknown")
+        _need(tau > 0, "tau must be positive")
+        _dense(z, "z", torch.float32, (rows, heads * dim))
+        _dense(bias, "bias", torch.float32, (heads * dim,))
+        _dense(state, "state", torch.float32, (state.shape[0], heads, dim, vdim))
+        _dense(out, "out", torch.float32, (rows, heads * vdim))
+        _dense(row_seg, "row_seg", torch.int32, (rows,))
+        _dense(seg_start, "seg_start", torch.int32)
+        _dense(slots, "slots", torch.int32)
+        num_segs = seg_start.numel() - 1
+        _need(num_segs >= 1 and slots.numel() >= num_segs, "gated_linear_attention: a slot a segment")
+        carried = None
+        if form != "tokens" and rows > num_segs:
+            need = int(self.lib.fllm_gated_linear_carried_floats(rows, num_segs, heads, dim, vdim))
+            carried = torch.empty((need,), dtype=torch.float32, device=qkv.device) if need else None
+        elem, base = qkv.element_size(), qkv.data_ptr()
+        self._check(self.lib.fllm_gated_linear_attention(
+            base, base + heads * dim * elem, base + 2 * heads * dim * elem, ld, _ptr(z), _ptr(bias), float(tau), float(query_scale), _ptr(state),
+            _ptr(row_seg), _ptr(seg_start), _ptr(slots), num_segs, _ptr(out), rows, heads, dim, vdim, {"auto": 0, "tokens": 1, "chunks": 2}[form],
+            _DTYPE_CODE[qkv.dtype], _ptr(carried), self._stream()))
+        return out
+
+    def min_recurrence(self, zxg: torch.Tensor, bias: torch.Tensor, state: torch.Tensor, row_seg: torch.Tensor, seg_start: torch.Tensor,
+                       slots: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+        """S <- (1 - z) S + z c lane by lane over each segment's rows [a | x | g] (three times out's width): z = sigmoid(a + bias[:width]),
+        u = x + bias[width:], c = u + 1/2 where u >= 0 and sigmoid(u) below; out = S * silu(g); S float32 state[slots, width]."""
+        rows, width = out.shape
+        _need(zxg.is_cuda and zxg.dim() == 2 and zxg.is_contiguous() and zxg.dtype in _DTYPE_CODE and tuple(zxg.shape) == (rows, 3 * width),
+              f"zxg must be dense rows of {3 * width} values on the GPU")
+        _dense(bias, "bias", torch.float32, (2 * width,))
+        _dense(state, "state", torch.float32, (state.shape[0], width))
+        _dense(out, "out", zxg.dtype)
+        _dense(row_seg, "row_seg", torch.int32, (rows,))
+        _dense(seg_start, "seg_start", torch.int32)
+        _dense(slots, "slots", torch.int32)
+        num_segs = seg_start.numel() - 1
+        _need(num_segs >= 1 and slots.numel() >= num_segs, "min_recurrence: a slot a segment")
+        need = int(self.lib.fllm_min_recurrence_carried_floats(rows, num_segs, width)) if rows > num_segs else 0
+        carried = torch.empty((need,), dtype=torch.float32, device=zxg.device) if need else None
+        self._check(self.lib.fllm_min_recurrence(_ptr(zxg), zxg.shape[1], _ptr(bias), _ptr(state), _ptr(row_seg), _ptr(seg_start), _ptr(slots),
+                                                 num_segs, _ptr(out), rows, width, _DTYPE_CODE[zxg.dtype], _ptr(carried), self._stream()))
+        return out
 
     def measured_ceilings(self, read_bytes: int = 4 << 30, repeats: int = 5) -> dict:
         """What the device delivers to kernels that do nothing else: GB/s of a kernel that only reads a buffer much larger
