@@ -409,16 +409,15 @@ int fllm_rotate_scale(const void *qkv, int ld, float *out, const int32_t *row_po
                       hipStream_t stream);
 // Softmax attention over the row's own chunk of `chunk` positions (window 0), or over its last `window` positions and the first
 // `keep_first` of the sequence (chunk 0; both 0: every position up to the row): score = q . k * scale, with softcap > 0 then
-// softcap * tanh(score / softcap); zero_sink: the denominator holds one more term exp(0) without a value.  spread 0: out of `dtype`
-// [rows, heads * v_dim]; spread 1: every head's weights meet the values of every key/value head, out float32 [rows, heads, kv_heads,
-// v_dim].  fllm_mix_heads: out_h = sum_g talk[h, g] * spread[g][h's key/value head] ([rows, heads * v_dim] of `dtype`), which is what
-// head h gets when the heads' WEIGHTS are mixed by talk (float32 [heads, heads]) before they meet the values.
+// softcap * tanh(score / softcap); zero_sink: the denominator holds one more term exp(0) without a value; out of `dtype` [rows, heads
+// * v_dim].  talk (float32 [heads, heads], or null): head h applies sum_g talk[h, g] (weights of head g) to the values of its own
+// key/value head: every head's weights meet the values of every key/value head (`spread`: float32 room of rows * heads * kv_heads *
+// v_dim), and the heads' results are mixed behind that.
 int fllm_masked_attention(const void *q, int q_stride, const void *k_pages, const void *v_pages, const int32_t *tables, int table_stride,
                           const int32_t *row_pos, const int32_t *row_seg, const int32_t *seg_start, int num_segs, void *out, int rows,
                           int heads, int kv_heads, int head_dim, int v_dim, int page_size, float scale, float softcap, int zero_sink,
-                          int chunk, int window, int keep_first, int spread, int key_chunk, int dtype, int max_context, hipStream_t stream);
-int fllm_mix_heads(const float *spread, const float *talk, void *out, int rows, int heads, int kv_heads, int v_dim, int dtype,
-                   hipStream_t stream);
+                          int chunk, int window, int keep_first, const float *talk, float *spread, int key_chunk, int dtype, int max_context,
+                          hipStream_t stream);
 // out = x / rms(x over each group of `group` lanes) * weight * act(gate), act silu or sigmoid, weight float32 [group] or null (1);
 // x float32 or of `dtype`.
 int fllm_group_norm_gate(const void *x, int x_dtype, const float *weight, float eps, int group, const void *gate, int gate_ld, void *out, int rows, int width,

@@ -1,0 +1,527 @@
+// Softmax attention over a row's own chunk of positions, or over a window and the sequence's first tokens, on the matrix cores
+// (bfloat16 pages, float32 scores and weights): capped scores, a sink of score 0, and heads whose weights meet the values of
+// several key/value heads.
+//
+// Both kernels compute the transposed products on v_mfma_f32_16x16x32_bf16, so that a lane keeps one query throughout:
+//   S^T = K Q^T      A = 16 keys x 32 lanes, B = Q^T.  A's row c of tile j of a 32-key block holds key (c / 4) * 8 + j * 4 + c % 4, so
+//                    that the two tiles leave lane group g = lane / 16 with the keys g * 8 .. g * 8 + 7 of its query in order,
+//   O^T += V^T P^T   which is how this product wants its B operand, and how a value lane's tokens lie in a page.
+// Weights stay float32: P goes into the product as the sum of two bfloat16 numbers (its rounding and what the rounding lost).
+//
+//   row tiles   portions of prompts: a workgroup of four waves takes 64 (token, head of the group) queries of one key/value head,
+//               16 a wave; keys and values go through LDS in tiles of 64, the next tile on its way while this one is multiplied.
+//   by heads    steps of single rows: a workgroup takes the heads of one key/value head of one row and a share of its keys, operands
+//               straight from the pages; a second kernel adds the shares, and mixes the heads where the design does.
+#include <algorithm>
+
+#include "api.h"
+#include "common.h"
+
+namespace {
+
+constexpr int kThreads = 256;
+constexpr int kWavesM = kThreads / kWave;
+constexpr float kLog2e = 1.4426950408889634f;
+
+struct MaskedParams {
+    const bf16_t *q;
+    int q_stride;
+    const bf16_t *k_pages, *v_pages;
+    const int32_t *tables;
+    int table_stride;
+    const int32_t *row_pos, *row_seg, *seg_start;
+    int num_segs;
+    void *out;                 // bfloat16 [row][head][DV], or float [row][head][kv_heads][DV] where values are spread
+    int rows, heads, kv_heads, page_size, ps_shift;
+    float scale_log2;          // scale * log2(e)
+    float cap_log2, cap_rate;  // cap * log2(e) and 2 * log2(e) * scale / cap; cap_log2 0: no cap
+    int zero_sink, chunk, window, keep_first, spread;
+    int splits;                // workgroups that share a row's keys (by heads)
+    float *parts;              // [row][key/value head][value group][split][16 * NV * DV sums, 16 maxima, 16 denominators]
+};
+
+__device__ __forceinline__ float fast_exp2(float x) { return __builtin_amdgcn_exp2f(x); }
+
+// the first position of the row's own range: of its window or its chunk; never falls as pos grows
+__device__ __forceinline__ int range_start(const MaskedParams &p, int pos) {
+    if (p.chunk > 0) return pos - pos % p.chunk;
+    return p.window > 0 && pos - p.window + 1 > 0 ? pos - p.window + 1 : 0;
+}
+
+// a product's value -> score in units of log2
+__device__ __forceinline__ float score_of(const MaskedParams &p, float dot) {
+    if (p.cap_log2 > 0.f)      // cap tanh(x / cap) = cap - 2 cap / (exp(2 x / cap) + 1): an overflowing exponential gives cap, none -cap
+        return p.cap_log2 - 2.0f * p.cap_log2 * __builtin_amdgcn_rcpf(fast_exp2(dot * p.cap_rate) + 1.0f);
+    return dot * p.scale_log2;
+}
+
+// The online softmax of 8 scores a lane (visible ones; others -inf): weights as two bfloat16 terms; the maximum is shared by a
+// query's four lane groups, the denominator stays the lane's own until the end.
+__device__ __forceinline__ float weigh8(const float (&s)[8], float m_new, bf16x8_t &hi, bf16x8_t &lo) {
+    float sum = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; e++) {
+        const float w = s[e] == -INFINITY ? 0.f : fast_exp2(s[e] - m_new);
+        sum += w;
+        hi[e] = (bf16_t)w;
+        lo[e] = (bf16_t)(w - (float)hi[e]);
+    }
+    return sum;
+}
+
+__device__ __forceinline__ bf16x8_t zero8() {
+    bf16x8_t z;
+#pragma unroll
+    for (int e = 0; e < 8; e++) z[e] = (bf16_t)0.f;
+    return z;
+}
+
+// ---- row tiles ----------------------------------------------------------------------------------------------------------------
+// grid ((row tiles, key/value head fastest), value groups).  NV: value heads a workgroup multiplies (its own one, or NV of all).
+template <int KD, int VT, int NV>
+__global__ void __launch_bounds__(kThreads, 2)
+masked_rows_kernel(const MaskedParams p) {
+    constexpr int D = KD * 32, DV = VT * 16, KT = 64, KP = D + 8, VP = KT + 8;
+    constexpr int KCH = KT * D / 8 / kThreads, VCH = NV * DV * KT / 8 / kThreads;      // 16-byte pieces a thread
+    static_assert(KT * D / 8 % kThreads == 0 && NV * DV * KT / 8 % kThreads == 0, "whole pieces a thread");
+    __shared__ __attribute__((aligned(16))) bf16_t Ks[KT * KP];
+    __shared__ __attribute__((aligned(16))) bf16_t Vs[NV * DV * VP];
+    __shared__ int s_tile[2];
+    const int G = p.heads / p.kv_heads, TQ = 64 / G;
+    const int kvh = blockIdx.x % p.kv_heads, vh0 = p.spread ? blockIdx.y * NV : kvh;
+    if (threadIdx.x == 0) {
+        int b = blockIdx.x / p.kv_heads, seg = -1, t0 = 0;
+        for (int s = 0; s < p.num_segs; s++) {
+            const int nt = (p.seg_start[s + 1] - p.seg_start[s] + TQ - 1) / TQ;
+            if (b < nt) {
+                seg = s;
+                t0 = nt - 1 - b;      // the tiles with the longest contexts start first
+                break;
+            }
+            b -= nt;
+        }
+        s_tile[0] = seg;
+        s_tile[1] = t0;
+    }
+    __syncthreads();
+    const int seg = s_tile[0];
+    if (seg < 0) return;
+    const int row0 = p.seg_start[seg] + s_tile[1] * TQ;
+    const int ntok = min(TQ, p.seg_start[seg + 1] - row0);
+    const int lane = threadIdx.x & (kWave - 1), wave = threadIdx.x / kWave;
+    const int c = lane & 15, g = lane >> 4;
+    const int qi = wave * 16 + c, tq = qi / G, head = kvh * G + (qi - tq * G);
+    const bool valid = tq < ntok && p.row_seg[row0] >= 0;
+    if (p.row_seg[row0] < 0) {      // padding rows: zeros
+        if (tq < ntok && g == 0)
+            for (int i = 0; i < NV * DV; i++) {
+                const size_t row = row0 + tq;
+                if (p.spread) ((float *)p.out)[((row * p.heads + head) * p.kv_heads + vh0) * DV + i] = 0.f;
+                else ((bf16_t *)p.out)[(row * p.heads + head) * DV + i] = (bf16_t)0.f;
+            }
+        return;
+    }
+    const int pos0 = p.row_pos[row0], pos_last = pos0 + ntok - 1;
+    const int my_pos = valid ? pos0 + tq : -1;
+    const int my_lo = valid ? range_start(p, my_pos) : 0;
+    const int32_t *tbl = p.tables + (size_t)seg * p.table_stride;
+    const int ps = p.page_size, psh = p.ps_shift, pmask = ps - 1;
+
+    bf16x8_t qf[KD];
+#pragma unroll
+    for (int kk = 0; kk < KD; kk++)
+        qf[kk] = valid ? *(const bf16x8_t *)(p.q + (size_t)(row0 + tq) * p.q_stride + (size_t)head * D + kk * 32 + g * 8) : zero8();
+
+    // the tile's key tiles: those of the first tokens that its window has passed, then from its first row's range on.  Positions
+    // that stand in both are visible in the second only.
+    const int lo_tile = range_start(p, pos0);                                  // smallest range start of the tile's rows
+    const int main0 = lo_tile & ~(KT - 1);
+    const int first_end = min(min(p.keep_first, range_start(p, pos_last)), main0);   // first-token tiles end before the others begin
+    const int first_tiles = (first_end + KT - 1) / KT;
+    const int tiles = first_tiles + (pos_last - main0) / KT + 1;
+    const int cps = psh < 6 ? psh - 3 : 3;       // log2 of the 8-token pieces of a value lane that lie together in a page and tile
+
+    bf16x8_t rk[KCH], rv[VCH];
+    auto tile_base = [&](int t) { return t < first_tiles ? t * KT : main0 + (t - first_tiles) * KT; };
+    auto issue = [&](int t) {
+        const int k0 = tile_base(t);
+#pragma unroll
+        for (int i = 0; i < KCH; i++) {
+            const int ch = threadIdx.x + i * kThreads, key = ch & (KT - 1), dc = ch / KT;
+            const int kabs = min(k0 + key, pos_last);      // keys behind the tile's last row: an address that exists; masked
+            rk[i] = *(const bf16x8_t *)(p.k_pages + key_offset(tbl[kabs >> psh], p.kv_heads, kvh, ps, D, kabs & pmask, dc * 8));
+        }
+#pragma unroll
+        for (int i = 0; i < VCH; i++) {
+            const int ch = threadIdx.x + i * kThreads;
+            const int nv = ch / (DV * KT / 8), r0 = ch - nv * (DV * KT / 8);
+            const int pg = r0 / (DV << cps), r1 = r0 - pg * (DV << cps);       // stretches of 8 << cps tokens
+            const int d = r1 >> cps, koff = (pg << (cps + 3)) + (r1 & ((1 << cps) - 1)) * 8;
+            const int kabs = k0 + koff;
+            bf16x8_t v = zero8();
+            if (kabs <= pos_last) {
+                v = *(const bf16x8_t *)(p.v_pages + (((size_t)tbl[kabs >> psh] * p.kv_heads + vh0 + nv) * DV + d) * ps + (kabs & pmask));
+                if (kabs + 7 > pos_last)      // slots past the last token hold whatever an earlier request left
+#pragma unroll
+                    for (int e = 0; e < 8; e++)
+                        if (kabs + e > pos_last) v[e] = (bf16_t)0.f;
+            }
+            rv[i] = v;
+        }
+    };
+    auto commit = [&]() {
+#pragma unroll
+        for (int i = 0; i < KCH; i++) {
+            const int ch = threadIdx.x + i * kThreads;
+            *(bf16x8_t *)(Ks + (ch & (KT - 1)) * KP + ch / KT * 8) = rk[i];
+        }
+#pragma unroll
+        for (int i = 0; i < VCH; i++) {
+            const int ch = threadIdx.x + i * kThreads;
+            const int nv = ch / (DV * KT / 8), r0 = ch - nv * (DV * KT / 8);
+            const int pg = r0 / (DV << cps), r1 = r0 - pg * (DV << cps);
+            const int d = r1 >> cps, koff = (pg << (cps + 3)) + (r1 & ((1 << cps) - 1)) * 8;
+            *(bf16x8_t *)(Vs + (nv * DV + d) * VP + koff) = rv[i];
+        }
+    };
+
+    f32x4_t o[NV * VT];
+#pragma unroll
+    for (int t = 0; t < NV * VT; t++) o[t] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+    float m_run = -INFINITY, l_run = 0.f;
+    issue(0);
+    for (int t = 0; t < tiles; t++) {
+        __syncthreads();      // the tile before has been read
+        commit();
+        if (t + 1 < tiles) issue(t + 1);
+        __syncthreads();
+        const int k0 = tile_base(t);
+        const bool firsts = t < first_tiles;
+        f32x4_t st[4];
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            st[i] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+            const int key_local = (i >> 1) * 32 + (c >> 2) * 8 + (i & 1) * 4 + (c & 3);
+#pragma unroll
+            for (int kk = 0; kk < KD; kk++) {
+                const bf16x8_t a = *(const bf16x8_t *)(Ks + key_local * KP + kk * 32 + g * 8);
+                st[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, qf[kk], st[i], 0, 0, 0);
+            }
+        }
+        float s[2][8];
+        float m_blk = -INFINITY;
+#pragma unroll
+        for (int b = 0; b < 2; b++)
+#pragma unroll
+            for (int e = 0; e < 8; e++) {
+                const int key = k0 + b * 32 + g * 8 + e;
+                const bool vis = key <= my_pos && (firsts ? key < p.keep_first && key < my_lo : key >= my_lo || key < p.keep_first) &&
+                                 (!firsts || key < first_end);
+                s[b][e] = vis ? score_of(p, st[b * 2 + (e >> 2)][e & 3]) : -INFINITY;
+                m_blk = fmaxf(m_blk, s[b][e]);
+            }
+        m_blk = fmaxf(m_blk, __shfl_xor(m_blk, 16, kWave));
+        m_blk = fmaxf(m_blk, __shfl_xor(m_blk, 32, kWave));
+        const float m_new = fmaxf(m_run, m_blk);
+        if (__any(m_new > m_run)) {      // the outputs are rescaled only when some row's maximum moved
+            const float alpha = m_run == -INFINITY ? 0.f : fast_exp2(m_run - m_new);
+            l_run *= alpha;
+#pragma unroll
+            for (int i = 0; i < NV * VT; i++) o[i] *= alpha;
+            m_run = m_new;
+        }
+#pragma unroll
+        for (int b = 0; b < 2; b++) {
+            bf16x8_t hi, lo;
+            l_run += weigh8(s[b], m_run, hi, lo);
+#pragma unroll
+            for (int i = 0; i < NV * VT; i++) {
+                const bf16x8_t a = *(const bf16x8_t *)(Vs + (i * 16 + c) * VP + b * 32 + g * 8);
+                o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, hi, o[i], 0, 0, 0);
+                o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, lo, o[i], 0, 0, 0);
+            }
+        }
+    }
+    l_run += __shfl_xor(l_run, 16, kWave);
+    l_run += __shfl_xor(l_run, 32, kWave);
+    if (!valid) return;
+    if (p.zero_sink) l_run += fast_exp2(-m_run);
+    const float inv = 1.0f / l_run;
+    const size_t row = row0 + tq;
+#pragma unroll
+    for (int i = 0; i < NV * VT; i++) {
+        const f32x4_t v = o[i] * inv;
+        if (p.spread) {
+            *(f32x4_t *)((float *)p.out + ((row * p.heads + head) * p.kv_heads + vh0) * DV + i * 16 + g * 4) = v;
+        } else {
+            bf16x4_t b;
+#pragma unroll
+            for (int e = 0; e < 4; e++) b[e] = (bf16_t)v[e];
+            *(bf16x4_t *)((bf16_t *)p.out + (row * p.heads + head) * DV + i * 16 + g * 4) = b;
+        }
+    }
+}
+
+// ---- by heads -------------------------------------------------------------------------------------------------------------------
+// grid (rows, key/value heads * value groups, splits); at most 16 heads a key/value head.  Blocks of 32 keys are dealt to the
+// workgroups' waves in turn; the waves meet in LDS and the workgroup leaves its share: sums against its own maximum.
+template <int KD, int VT, int NV>
+__global__ void __launch_bounds__(kThreads)
+masked_heads_kernel(const MaskedParams p) {
+    constexpr int D = KD * 32, DV = VT * 16, W = NV * DV;
+    __shared__ float sm_o[kWavesM][16][DV + 1];      // one value head at a time
+    __shared__ float sm_m[kWavesM][16], sm_l[kWavesM][16];
+    const int row = blockIdx.x, seg = p.row_seg[row];
+    if (seg < 0) return;      // padding row: the merge writes its zeros
+    const int G = p.heads / p.kv_heads;
+    const int kvh = blockIdx.y % p.kv_heads, vh0 = p.spread ? blockIdx.y / p.kv_heads * NV : kvh;
+    const int lane = threadIdx.x & (kWave - 1), wave = threadIdx.x / kWave;
+    const int qi = lane & 15, g = lane >> 4;
+    const bool valid = qi < G;
+    const int pos = p.row_pos[row], lo = range_start(p, pos);
+    const int32_t *tbl = p.tables + (size_t)seg * p.table_stride;
+    const int ps = p.page_size, psh = p.ps_shift, pmask = ps - 1;
+    bf16x8_t qf[KD];
+#pragma unroll
+    for (int kk = 0; kk < KD; kk++)
+        qf[kk] = valid ? *(const bf16x8_t *)(p.q + (size_t)row * p.q_stride + (size_t)(kvh * G + qi) * D + kk * 32 + g * 8) : zero8();
+    f32x4_t o[NV * VT];
+#pragma unroll
+    for (int t = 0; t < NV * VT; t++) o[t] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+    float m_run = -INFINITY, l_run = 0.f;
+    const int main0 = lo & ~31, first_end = min(min(p.keep_first, lo), main0);
+    const int first_blocks = (first_end + 31) / 32, blocks = first_blocks + (pos - main0) / 32 + 1;
+    for (int b = blockIdx.z * kWavesM + wave; b < blocks; b += p.splits * kWavesM) {
+        const bool firsts = b < first_blocks;
+        const int base = firsts ? b * 32 : main0 + (b - first_blocks) * 32;
+        bf16x8_t ka[2][KD], va[NV * VT];
+#pragma unroll
+        for (int j = 0; j < 2; j++) {
+            const int key = min(base + (qi >> 2) * 8 + j * 4 + (qi & 3), pos);
+            const bf16_t *kr = p.k_pages + key_offset(tbl[key >> psh], p.kv_heads, kvh, ps, D, key & pmask, g * 8);
+#pragma unroll
+            for (int kk = 0; kk < KD; kk++) ka[j][kk] = *(const bf16x8_t *)(kr + (size_t)kk * 4 * ps * 8);
+        }
+        {
+            int key = base + g * 8;      // eight tokens side by side in one page
+            key = key <= pos ? key : pos & ~7;
+            const bf16_t *vr = p.v_pages + (((size_t)tbl[key >> psh] * p.kv_heads + vh0) * DV + qi) * ps + (key & pmask);
+#pragma unroll
+            for (int t = 0; t < NV * VT; t++) va[t] = *(const bf16x8_t *)(vr + (size_t)t * 16 * ps);      // value heads lie one behind the other
+        }
+        f32x4_t st[2];
+#pragma unroll
+        for (int j = 0; j < 2; j++) {
+            st[j] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int kk = 0; kk < KD; kk++) st[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ka[j][kk], qf[kk], st[j], 0, 0, 0);
+        }
+        float s[8];
+        float m_blk = -INFINITY;
+#pragma unroll
+        for (int e = 0; e < 8; e++) {
+            const int key = base + g * 8 + e;
+            const bool vis = key <= pos && (firsts ? key < first_end : key >= lo || key < p.keep_first);
+            s[e] = vis ? score_of(p, st[e >> 2][e & 3]) : -INFINITY;
+            m_blk = fmaxf(m_blk, s[e]);
+        }
+        if (base + 31 > pos)      // slots past the last token hold whatever an earlier request left: a weight of 0 must meet a number
+#pragma unroll
+            for (int e = 0; e < 8; e++)
+                if (base + g * 8 + e > pos)
+#pragma unroll
+                    for (int t = 0; t < NV * VT; t++) va[t][e] = (bf16_t)0.f;
+        m_blk = fmaxf(m_blk, __shfl_xor(m_blk, 16, kWave));
+        m_blk = fmaxf(m_blk, __shfl_xor(m_blk, 32, kWave));
+        const float m_new = fmaxf(m_run, m_blk);
+        const float alpha = m_run == -INFINITY ? 0.f : fast_exp2(m_run - m_new);
+        bf16x8_t hi, lo8;
+        l_run = l_run * alpha + (m_new == -INFINITY ? 0.f : weigh8(s, m_new, hi, lo8));
+        if (m_new == -INFINITY) hi = lo8 = zero8();
+        m_run = m_new;
+#pragma unroll
+        for (int t = 0; t < NV * VT; t++) {
+            o[t] *= alpha;
+            o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(va[t], hi, o[t], 0, 0, 0);
+            o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(va[t], lo8, o[t], 0, 0, 0);
+        }
+    }
+    l_run += __shfl_xor(l_run, 16, kWave);
+    l_run += __shfl_xor(l_run, 32, kWave);
+    if (g == 0) sm_m[wave][qi] = m_run, sm_l[wave][qi] = l_run;
+    float *part = p.parts + (((size_t)row * gridDim.y + blockIdx.y) * p.splits + blockIdx.z) * (16 * W + 32);
+#pragma unroll
+    for (int nv = 0; nv < NV; nv++) {
+        if (nv > 0) __syncthreads();
+#pragma unroll
+        for (int t = 0; t < VT; t++)
+#pragma unroll
+            for (int i = 0; i < 4; i++) sm_o[wave][qi][t * 16 + g * 4 + i] = o[nv * VT + t][i];
+        __syncthreads();
+        for (int idx = threadIdx.x; idx < G * DV; idx += kThreads) {
+            const int q = idx / DV, d = idx - q * DV;
+            float m = -INFINITY, l = 0.f, acc = 0.f;
+#pragma unroll
+            for (int w = 0; w < kWavesM; w++) m = fmaxf(m, sm_m[w][q]);
+#pragma unroll
+            for (int w = 0; w < kWavesM; w++) {
+                const float f = sm_m[w][q] == -INFINITY ? 0.f : fast_exp2(sm_m[w][q] - m);
+                l += sm_l[w][q] * f;
+                acc += sm_o[w][q][d] * f;
+            }
+            part[q * W + nv * DV + d] = acc;
+            if (nv == 0 && d == 0) part[16 * W + q] = m, part[16 * W + 16 + q] = l;
+        }
+    }
+}
+
+// The shares put together in their order: grid (rows, key/value heads of the outputs).  Without `talk` the workgroup writes its key/value
+// head's outputs; with it, it gathers what every head's weights made of this key/value head's values and mixes: out_h = sum_g
+// talk[h][g] A_g.  LDS: heads * DV floats and a factor a head and split.
+__global__ void __launch_bounds__(kThreads)
+masked_merge_kernel(const float *__restrict__ parts, int splits, const int32_t *__restrict__ row_seg, const float *__restrict__ talk,
+                    bf16_t *__restrict__ out, int heads, int kv_heads, int DV, int NV, int zero_sink) {
+    extern __shared__ float smem[];
+    const int row = blockIdx.x, vh = blockIdx.y, G = heads / kv_heads;
+    bf16_t *dst = out + ((size_t)row * heads + vh * G) * DV;
+    if (row_seg[row] < 0) {      // padding row: zeros
+        for (int i = threadIdx.x; i < G * DV; i += kThreads) dst[i] = (bf16_t)0.f;
+        return;
+    }
+    const int count = talk != nullptr ? heads : G, first = talk != nullptr ? 0 : vh * G;      // heads whose shares this workgroup reads
+    float *factor = smem;                       // [count][splits]
+    float *A = factor + count * splits;         // [count][DV]
+    const int W = NV * DV, stride = 16 * W + 32;
+    const int groups = talk != nullptr ? kv_heads / NV : 1, at = talk != nullptr ? vh % NV : 0;
+    const int ny = kv_heads * groups, yv = talk != nullptr ? vh / NV : 0;
+    auto share = [&](int h, int s) {
+        const int kvh = h / G;
+        return parts + (((size_t)row * ny + yv * kv_heads + kvh) * splits + s) * stride;
+    };
+    for (int i = threadIdx.x; i < count; i += kThreads) {
+        const int h = first + i, q = h % G;
+        float m = -INFINITY, l = 0.f;
+        for (int s = 0; s < splits; s++) m = fmaxf(m, share(h, s)[16 * W + q]);
+        for (int s = 0; s < splits; s++) {
+            const float ms = share(h, s)[16 * W + q];
+            const float f = ms == -INFINITY ? 0.f : fast_exp2(ms - m);
+            l += share(h, s)[16 * W + 16 + q] * f;
+            factor[i * splits + s] = f;
+        }
+        if (zero_sink) l += fast_exp2(-m);
+        const float inv = 1.0f / l;
+        for (int s = 0; s < splits; s++) factor[i * splits + s] *= inv;
+    }
+    __syncthreads();
+    for (int idx = threadIdx.x; idx < count * DV; idx += kThreads) {
+        const int i = idx / DV, d = idx - i * DV, h = first + i, q = h % G;
+        float acc = 0.f;
+#pragma unroll 4
+        for (int s = 0; s < splits; s++) acc = fmaf(share(h, s)[q * W + at * DV + d], factor[i * splits + s], acc);
+        if (talk == nullptr) dst[idx] = (bf16_t)acc;
+        else A[idx] = acc;
+    }
+    if (talk == nullptr) return;
+    __syncthreads();
+    for (int idx = threadIdx.x; idx < G * DV; idx += kThreads) {
+        const int hl = idx / DV, d = idx - hl * DV;
+        const float *tk = talk + (size_t)(vh * G + hl) * heads;
+        float acc = 0.f;
+        for (int g = 0; g < heads; g++) acc = fmaf(tk[g], A[g * DV + d], acc);
+        dst[idx] = (bf16_t)acc;
+    }
+}
+
+template <int KD, int VT, int NV>
+void launch_one(const MaskedParams &p, bool by_heads, dim3 grid, hipStream_t stream) {
+    if (by_heads) hipLaunchKernelGGL((masked_heads_kernel<KD, VT, NV>), grid, dim3(kThreads), 0, stream, p);
+    else hipLaunchKernelGGL((masked_rows_kernel<KD, VT, NV>), grid, dim3(kThreads), 0, stream, p);
+}
+
+template <int KD, int NV>
+void launch_vt(const MaskedParams &p, int vt, bool by_heads, dim3 grid, hipStream_t stream) {
+    switch (vt) {
+    case 2: launch_one<KD, 2, NV>(p, by_heads, grid, stream); break;
+    case 4: launch_one<KD, 4, NV>(p, by_heads, grid, stream); break;
+    case 6: launch_one<KD, 6, NV>(p, by_heads, grid, stream); break;
+    case 8: launch_one<KD, 8, NV>(p, by_heads, grid, stream); break;
+    }
+}
+
+}  // namespace
+
+// 0: launched; 1: the shape is not one these kernels take (the caller runs the plain kernel).  Takes bfloat16 pages with keys in
+// chunks of 8, heads of 32, 64, 96 or 128 lanes and values of the same, pages of a power of two of at least 8 tokens, at most 64 heads
+// a key/value head (16 in steps of single rows).  talk (null: none): heads are mixed; then `spread` is float32 room of rows * heads *
+// kv_heads * v_dim for steps of portions (*mixed is set to 0: the caller mixes from there), steps of single rows mix by themselves
+// (*mixed 1).
+int fllm_masked_attention_bf16_fast(const void *q, int q_stride, const void *k_pages, const void *v_pages, const int32_t *tables,
+                                    int table_stride, const int32_t *row_pos, const int32_t *row_seg, const int32_t *seg_start,
+                                    int num_segs, void *out, int rows, int heads, int kv_heads, int head_dim, int v_dim, int page_size,
+                                    float scale, float softcap, int zero_sink, int chunk, int window, int keep_first, const float *talk,
+                                    float *spread, int *mixed, int max_context, hipStream_t stream) {
+    if (!fllm_fast_kernels_enabled() || seg_start == nullptr || num_segs <= 0) return 1;
+    if (head_dim % 32 != 0 || head_dim > 128 || v_dim % 32 != 0 || v_dim > 128) return 1;
+    if (page_size < 8 || (page_size & (page_size - 1)) != 0 || q_stride % 8 != 0 || ((uintptr_t)q & 15) != 0) return 1;
+    const int G = heads / kv_heads;
+    const bool by_heads = rows == num_segs;
+    if (G > (by_heads ? 16 : 64)) return 1;
+    MaskedParams p = {};
+    p.q = (const bf16_t *)q, p.q_stride = q_stride, p.k_pages = (const bf16_t *)k_pages, p.v_pages = (const bf16_t *)v_pages;
+    p.tables = tables, p.table_stride = table_stride, p.row_pos = row_pos, p.row_seg = row_seg, p.seg_start = seg_start;
+    p.num_segs = num_segs, p.rows = rows, p.heads = heads, p.kv_heads = kv_heads, p.page_size = page_size;
+    while ((1 << p.ps_shift) < page_size) p.ps_shift++;
+    p.scale_log2 = scale * kLog2e;
+    if (softcap > 0.f) p.cap_log2 = softcap * kLog2e, p.cap_rate = 2.0f * kLog2e * scale / softcap;
+    p.zero_sink = zero_sink, p.chunk = chunk, p.window = window, p.keep_first = keep_first;
+    p.spread = talk != nullptr;
+    p.out = talk != nullptr ? (void *)spread : out;
+    p.splits = 1;
+    const int NV = talk != nullptr && kv_heads % 2 == 0 ? 2 : 1;
+    const int groups = talk != nullptr ? kv_heads / NV : 1;
+    dim3 grid;
+    if (by_heads) {
+        // few rows: several workgroups share a row's keys (128 of them at least, two workgroups a compute unit at most)
+        int span = max_context > 0 ? max_context : 1 << 20;
+        if (chunk > 0) span = std::min(span, chunk);
+        if (window > 0) span = std::min(span, window + keep_first + 64);
+        const long tiles = (long)rows * kv_heads * groups;
+        long splits = std::max(1L, std::min(std::min(512 / std::max(tiles, 1L), (long)(span + 127) / 128), 32L));
+        void *base = nullptr;
+        size_t bytes = 0;
+        if (!fllm_device_workspace(&base, &bytes) || bytes <= kWorkspaceCounterBytes) return 1;
+        const size_t room = (bytes - kWorkspaceCounterBytes) / sizeof(float), each = (size_t)tiles * (16 * NV * v_dim + 32);
+        splits = std::min<long>(splits, (long)(room / each));
+        if (splits < 1) return 1;
+        const size_t smem = (size_t)(talk != nullptr ? heads : G) * (splits + v_dim) * sizeof(float);
+        if (smem > 64 * 1024) return 1;
+        p.splits = (int)splits;
+        p.parts = (float *)((char *)base + kWorkspaceCounterBytes);
+        grid = dim3(rows, kv_heads * groups, (unsigned)splits);
+        if (grid.y > 65535) return 1;
+    } else {
+        const int TQ = 64 / G;
+        grid = dim3((unsigned)(((rows + TQ - 1) / TQ + num_segs) * kv_heads), groups);
+        if (groups > 65535) return 1;
+    }
+#define FLLM_KD(KD)                                                                     \
+    do {                                                                                \
+        if (NV == 2) launch_vt<KD, 2>(p, v_dim / 16, by_heads, grid, stream);           \
+        else launch_vt<KD, 1>(p, v_dim / 16, by_heads, grid, stream);                   \
+    } while (0)
+    switch (head_dim / 32) {
+    case 1: FLLM_KD(1); break;
+    case 2: FLLM_KD(2); break;
+    case 3: FLLM_KD(3); break;
+    case 4: FLLM_KD(4); break;
+    }
+#undef FLLM_KD
+    *mixed = 0;
+    if (by_heads) {
+        const size_t smem = (size_t)(talk != nullptr ? heads : G) * (p.splits + v_dim) * sizeof(float);
+        hipLaunchKernelGGL(masked_merge_kernel, dim3(rows, kv_heads), dim3(kThreads), smem, stream, p.parts, p.splits, row_seg, talk, (bf16_t *)out,
+                           heads, kv_heads, v_dim, NV, zero_sink);
+        *mixed = 1;
+    }
+    return fllm_check_launch("masked_attention (matrix cores)");
+}

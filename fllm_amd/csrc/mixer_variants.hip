@@ -10,9 +10,9 @@
 //                            before them; one softmax over both kinds.
 //   sigmoid_attention        no softmax: key j weighs sigmoid(cap * tanh(s / cap) - r1 ln(1 + r2 (pos - j)) + pb) on its own.
 //   masked_attention         softmax over the row's own chunk of positions, or over a window and the sequence's first tokens; scores
-//                            capped where asked, one more term of score 0 in the denominator where asked; a head's weights meet
-//                            the values of its own key/value head, or (spread) of every key/value head.
-//   mix_heads                out_h = sum_g talk[h][g] (head g's weights times the values of h's key/value head).
+//                            capped where asked, one more term of score 0 in the denominator where asked.  Heads whose WEIGHTS are
+//                            mixed before they meet the values: every head's weights meet the values of every key/value head
+//                            (float32), and out_h = sum_g talk[h][g] (head g's weights times the values of h's key/value head).
 //   rotate_scale             q and k of a linear attention rotated and k scaled, in float32, values beside them.
 //   group_norm_gate          every group of lanes divided by its root mean square, times a weight a lane of a group where there is
 //                            one, times silu or sigmoid of a gate.
@@ -37,8 +37,8 @@ int fllm_sigmoid_attention_bf16_fast(const void *q, int q_stride, const void *k_
 int fllm_masked_attention_bf16_fast(const void *q, int q_stride, const void *k_pages, const void *v_pages, const int32_t *tables,
                                     int table_stride, const int32_t *row_pos, const int32_t *row_seg, const int32_t *seg_start,
                                     int num_segs, void *out, int rows, int heads, int kv_heads, int head_dim, int v_dim, int page_size,
-                                    float scale, float softcap, int zero_sink, int chunk, int window, int keep_first, int spread,
-                                    int max_context, hipStream_t stream);
+                                    float scale, float softcap, int zero_sink, int chunk, int window, int keep_first, const float *talk,
+                                    float *spread, int *mixed, int max_context, hipStream_t stream);   // masked_attention_mfma.hip
 
 namespace {
 
@@ -420,8 +420,8 @@ sigmoid_attention_kernel(const T *__restrict__ q, int q_stride, const T *__restr
 }
 
 // ---- softmax over a chunk, or over a window and the first tokens ---------------------------------------------------------------
-// grid (rows, heads, spread ? kv_heads : 1).  The row's keys in one line: the first tokens 0 .. nf - 1 that the window has passed,
-// then the positions lo .. pos.  O: T, or float with `spread` (out[row][head][value head][v_dim]).
+// grid (rows, heads, value heads a head's weights meet: 1 or all).  The row's keys in one line: the first tokens 0 .. nf - 1 that the window has passed,
+// then the positions lo .. pos.  O: T, or float where values are spread (out[row][head][value head][v_dim]).
 template <typename T, typename O>
 __global__ void __launch_bounds__(kBlock)
 masked_attention_kernel(const T *__restrict__ q, int q_stride, const T *__restrict__ k_pages, const T *__restrict__ v_pages,
@@ -739,8 +739,8 @@ extern "C" int fllm_sigmoid_attention(const void *q, int q_stride, const void *k
 extern "C" int fllm_masked_attention(const void *q, int q_stride, const void *k_pages, const void *v_pages, const int32_t *tables, int table_stride,
                                      const int32_t *row_pos, const int32_t *row_seg, const int32_t *seg_start, int num_segs, void *out,
                                      int rows, int heads, int kv_heads, int head_dim, int v_dim, int page_size, float scale, float softcap,
-                                     int zero_sink, int chunk, int window, int keep_first, int spread, int key_chunk, int dtype,
-                                     int max_context, hipStream_t stream) {
+                                     int zero_sink, int chunk, int window, int keep_first, const float *talk, float *spread, int key_chunk,
+                                     int dtype, int max_context, hipStream_t stream) {
     FLLM_REQUIRE(rows >= 0 && heads > 0 && heads <= 65535 && kv_heads > 0 && kv_heads <= 65535 && head_dim > 0 && v_dim > 0 && page_size > 0 &&
                      table_stride > 0, "masked_attention: bad sizes");
     FLLM_REQUIRE(softcap >= 0.f && chunk >= 0 && window >= 0 && keep_first >= 0 && (chunk == 0 || window == 0) && (keep_first == 0 || window > 0),
@@ -750,38 +750,44 @@ extern "C" int fllm_masked_attention(const void *q, int q_stride, const void *k_
     FLLM_REQUIRE(v_dim <= kBlock * kMaxLanes, "masked_attention: values of %d lanes a head are more than %d", v_dim, kBlock * kMaxLanes);
     FLLM_REQUIRE(q_stride >= heads * head_dim, "masked_attention: q_stride %d is shorter than heads * head_dim", q_stride);
     FLLM_REQUIRE(q && k_pages && v_pages && tables && row_pos && row_seg && out, "masked_attention: operands missing");
+    FLLM_REQUIRE(talk == nullptr || spread != nullptr, "masked_attention: heads that are mixed need room for their spread values");
     if (rows == 0) return 0;
+    const dim3 mix_grid(rows, (heads * v_dim + kBlock - 1) / kBlock);
+    FLLM_REQUIRE(mix_grid.y <= 65535, "masked_attention: too many heads");
+    auto mix = [&]() {
+        if (dtype == FLLM_F32)
+            hipLaunchKernelGGL(mix_heads_kernel<float>, mix_grid, dim3(kBlock), 0, stream, spread, talk, (float *)out, heads, kv_heads, v_dim);
+        else
+            hipLaunchKernelGGL(mix_heads_kernel<bf16_t>, mix_grid, dim3(kBlock), 0, stream, spread, talk, (bf16_t *)out, heads, kv_heads, v_dim);
+    };
     if (dtype == FLLM_BF16 && key_chunk == 8) {
+        int mixed = 0;
         const int fast = fllm_masked_attention_bf16_fast(q, q_stride, k_pages, v_pages, tables, table_stride, row_pos, row_seg, seg_start,
                                                          num_segs, out, rows, heads, kv_heads, head_dim, v_dim, page_size, scale, softcap,
-                                                         zero_sink, chunk, window, keep_first, spread, max_context, stream);
+                                                         zero_sink, chunk, window, keep_first, talk, spread, &mixed, max_context, stream);
+        if (fast == 0 && talk != nullptr && !mixed) {
+            mix();
+            return fllm_check_launch("mix_heads");
+        }
         if (fast <= 0) return fast;
     }
     const int vd_pad = pow2_lanes(v_dim);
     const size_t smem = (size_t)(((head_dim + 1) & ~1) + kBlock + 2 * ((kWaves + 1) / 2)) * sizeof(float) + (size_t)kBlock * (sizeof(long long) + sizeof(int)) +
                         (size_t)kMaxLanes * kBlock * sizeof(float);
     FLLM_REQUIRE(smem <= 64 * 1024, "masked_attention: heads of %d lanes do not fit into LDS", head_dim);
-    const dim3 grid(rows, heads, spread ? kv_heads : 1);
-#define FLLM_MASKED(T, O)                                                                                                                  hipLaunchKernelGGL((masked_attention_kernel<T, O>), grid, dim3(kBlock), smem, stream, (const T *)q, q_stride, (const T *)k_pages,                          (const T *)v_pages, tables, table_stride, row_pos, row_seg, (O *)out, heads, kv_heads, head_dim, v_dim, page_size,                        scale, softcap, zero_sink, chunk, window, keep_first, key_chunk, vd_pad)
+    const dim3 grid(rows, heads, talk != nullptr ? kv_heads : 1);
+    void *dst = talk != nullptr ? (void *)spread : out;
+#define FLLM_MASKED(T, O)                                                                                                               \
+    hipLaunchKernelGGL((masked_attention_kernel<T, O>), grid, dim3(kBlock), smem, stream, (const T *)q, q_stride, (const T *)k_pages,    \
+                       (const T *)v_pages, tables, table_stride, row_pos, row_seg, (O *)dst, heads, kv_heads, head_dim, v_dim,           \
+                       page_size, scale, softcap, zero_sink, chunk, window, keep_first, key_chunk, vd_pad)
     if (dtype == FLLM_F32) FLLM_MASKED(float, float);
-    else if (dtype == FLLM_BF16 && spread) FLLM_MASKED(bf16_t, float);
+    else if (dtype == FLLM_BF16 && talk != nullptr) FLLM_MASKED(bf16_t, float);
     else if (dtype == FLLM_BF16) FLLM_MASKED(bf16_t, bf16_t);
     else FLLM_REQUIRE(false, "masked_attention: unknown dtype %d", dtype);
 #undef FLLM_MASKED
+    if (talk != nullptr) mix();
     return fllm_check_launch("masked_attention");
-}
-
-extern "C" int fllm_mix_heads(const float *spread, const float *talk, void *out, int rows, int heads, int kv_heads, int v_dim, int dtype,
-                              hipStream_t stream) {
-    FLLM_REQUIRE(rows >= 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && v_dim > 0, "mix_heads: bad sizes");
-    FLLM_REQUIRE(spread && talk && out, "mix_heads: operands missing");
-    if (rows == 0) return 0;
-    const dim3 grid(rows, (heads * v_dim + kBlock - 1) / kBlock);
-    FLLM_REQUIRE(grid.y <= 65535, "mix_heads: too many heads");
-    if (dtype == FLLM_F32) hipLaunchKernelGGL(mix_heads_kernel<float>, grid, dim3(kBlock), 0, stream, spread, talk, (float *)out, heads, kv_heads, v_dim);
-    else if (dtype == FLLM_BF16) hipLaunchKernelGGL(mix_heads_kernel<bf16_t>, grid, dim3(kBlock), 0, stream, spread, talk, (bf16_t *)out, heads, kv_heads, v_dim);
-    else FLLM_REQUIRE(false, "mix_heads: unknown dtype %d", dtype);
-    return fllm_check_launch("mix_heads");
 }
 
 extern "C" int fllm_rotate_scale(const void *qkv, int ld, float *out, const int32_t *row_pos, const float *cos_table,

@@ -440,7 +440,3 @@ int fllm_sigmoid_attention_bf16_fast(const void *q, int q_stride, const void *k_
     if (launch_tiles<1>(p, head_dim, v_dim, max_context, stream)) return 1;
     return fllm_check_launch("sigmoid_attention (matrix cores)");
 }
-
-int fllm_masked_attention_bf16_fast(const void *, int, const void *, const void *, const int32_t *, int, const int32_t *, const int32_t *,
-                                    const int32_t *, int, void *, int, int, int, int, int, int, float, float, int, int, int, int, int, int,
-                                    hipStream_t) { return 1; }

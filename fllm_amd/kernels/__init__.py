@@ -157,8 +157,8 @@ def load_library(build_if_missing: bool = True):
                                 c_int, c_void, c_int, c_void, c_void, c_int, c_void, c_void, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
                                 c_int, c_int, c_int, c_int, c_int, c_void],
         "fllm_masked_attention": [c_void, c_int, c_void, c_void, c_void, c_int, c_void, c_void, c_void, c_int, c_void, c_int, c_int, c_int,
-                                  c_int, c_int, c_int, c_float, c_float, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void],
-        "fllm_mix_heads": [c_void, c_void, c_void, c_int, c_int, c_int, c_int, c_int, c_void],
+                                  c_int, c_int, c_int, c_float, c_float, c_int, c_int, c_int, c_int, c_void, c_void, c_int, c_int, c_int,
+                                  c_void],
         "fllm_gated_linear_attention": [c_void, c_void, c_void, c_int, c_void, c_void, c_float, c_float, c_void, c_void, c_void, c_void, c_int,
                                         c_void, c_int, c_int, c_int, c_int, c_int, c_int, c_void, c_void],
         "fllm_min_recurrence": [c_void, c_int, c_void, c_void, c_void, c_void, c_void, c_int, c_void, c_int, c_int, c_int, c_void, c_void],
@@ -1532,11 +1532,11 @@ class Ops:
     def masked_attention(self, q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, tables: torch.Tensor, row_pos: torch.Tensor,
                          row_seg: torch.Tensor, seg_start: torch.Tensor, out: torch.Tensor, heads: int, kv_heads: int, k_dim: int, v_dim: int,
                          page_size: int, scale: float, key_chunk: int, chunk: int = 0, window: int = 0, keep_first: int = 0,
-                         softcap: float = 0.0, zero_sink: bool = False, spread: bool = False, max_context: int = 0) -> torch.Tensor:
+                         softcap: float = 0.0, zero_sink: bool = False, talk: Optional[torch.Tensor] = None, max_context: int = 0) -> torch.Tensor:
         """Softmax attention over the row's own chunk of `chunk` positions, or over its last `window` positions and the first
         `keep_first` of the sequence (both 0: everything up to the row); `softcap` > 0: softcap * tanh(score / softcap);
-        `zero_sink`: one more term exp(0) in the denominator.  `spread`: a head's weights meet the values of every key/value head,
-        out float32 [rows, heads * kv_heads * v_dim] (for `mix_heads`)."""
+        `zero_sink`: one more term exp(0) in the denominator.  `talk` (float32 [heads, heads]): head h applies sum_g talk[h, g] *
+        (weights of head g) to the values of its own key/value head."""
         rows = q.shape[0]
         _need(q.is_cuda and q.dim() == 2 and q.stride(1) == 1 and q.shape[1] == heads * k_dim and q.dtype in _DTYPE_CODE,
               f"q must be [rows, {heads * k_dim}] of float32 or bfloat16 with unit column stride")
@@ -1546,24 +1546,17 @@ class Ops:
         _need(tables.dim() == 2, "tables must be [segments, pages]")
         _dense(row_pos, "row_pos", torch.int32, (rows,))
         _dense(row_seg, "row_seg", torch.int32, (rows,))
-        _dense(out, "out", *((torch.float32, (rows, heads * kv_heads * v_dim)) if spread else (q.dtype, (rows, heads * v_dim))))
+        _dense(out, "out", q.dtype, (rows, heads * v_dim))
         self._segments(seg_start, tables, rows)
+        spread = None
+        if talk is not None:      # what every head's weights make of every key/value head's values, until the heads are mixed
+            _dense(talk, "talk", torch.float32, (heads, heads))
+            spread = torch.empty((rows * heads * kv_heads * v_dim,), dtype=torch.float32, device=q.device)
         self._check(self.lib.fllm_masked_attention(
             _ptr(q), q.stride(0) if rows > 1 else heads * k_dim, _ptr(k_pages), _ptr(v_pages), _ptr(tables), tables.shape[1], _ptr(row_pos),
             _ptr(row_seg), _ptr(seg_start), seg_start.numel() - 1, _ptr(out), rows, heads, kv_heads, k_dim, v_dim, page_size, float(scale),
-            float(softcap), 1 if zero_sink else 0, int(chunk), int(window), int(keep_first), 1 if spread else 0, key_chunk,
+            float(softcap), 1 if zero_sink else 0, int(chunk), int(window), int(keep_first), _ptr(talk), _ptr(spread), key_chunk,
             _DTYPE_CODE[q.dtype], int(max_context), self._stream()))
-        return out
-
-    def mix_heads(self, spread: torch.Tensor, talk: torch.Tensor, out: torch.Tensor, heads: int, kv_heads: int, v_dim: int) -> torch.Tensor:
-        """out_h = sum_g talk[h, g] * spread[g][h's key/value head]; spread float32 [rows, heads * kv_heads * v_dim]."""
-        rows = out.shape[0]
-        _dense(spread, "spread", torch.float32, (rows, heads * kv_heads * v_dim))
-        _dense(talk, "talk", torch.float32, (heads, heads))
-        _dense(out, "out", None, (rows, heads * v_dim))
-        _need(out.dtype in _DTYPE_CODE, f"out dtype {out.dtype} unsupported")
-        self._check(self.lib.fllm_mix_heads(_ptr(spread), _ptr(talk), _ptr(out), rows, heads, kv_heads, v_dim, _DTYPE_CODE[out.dtype],
-                                            self._stream()))
         return out
 
     def gated_linear_attention(self, qkv: torch.Tensor, z: torch.Tensor, bias: torch.Tensor, tau: float, query_scale: float,

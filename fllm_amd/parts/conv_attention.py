@@ -124,15 +124,9 @@ class ConvAttention(Mixer):
                            single_rows=bool(ctx.uniform_rows))
         out = rt.empty((rows, nh * dv))
         mask = dict(chunk=self.chunk, window=self.window, keep_first=self.keep_first, softcap=self.softcap, zero_sink=self.zero_sink,
-                    max_context=ctx.max_context)
-        if self.talk is not None:
-            spread = rt.empty((rows, nh * nkv * dv), torch.float32)
-            ops.masked_attention(q, binding.k_pages, binding.v_pages, tables, ctx.row_pos, ctx.row_seg, ctx.seg_start, spread, nh, nkv, d, dv,
-                                 binding.page_size, self.scale, self.key_chunk, spread=True, **mask)
-            ops.mix_heads(spread, self.talk, out, nh, nkv, dv)
-        else:
-            ops.masked_attention(q, binding.k_pages, binding.v_pages, tables, ctx.row_pos, ctx.row_seg, ctx.seg_start, out, nh, nkv, d, dv,
-                                 binding.page_size, self.scale, self.key_chunk, **mask)
+                    talk=self.talk, max_context=ctx.max_context)
+        ops.masked_attention(q, binding.k_pages, binding.v_pages, tables, ctx.row_pos, ctx.row_seg, ctx.seg_start, out, nh, nkv, d, dv,
+                             binding.page_size, self.scale, self.key_chunk, **mask)
         if self.gated:
             gated = rt.empty((rows, nh * dv))
             out = ops.gated_norm(out, None, 0.0, joint[:, self.gate_at:], gated)

@@ -602,7 +602,7 @@ class ReferenceOps:
         return q_out
 
     def masked_attention(self, q, k_pages, v_pages, tables, row_pos, row_seg, seg_start, out, heads, kv_heads, k_dim, v_dim, page_size,
-                         scale, key_chunk, chunk=0, window=0, keep_first=0, softcap=0.0, zero_sink=False, spread=False, max_context=0):
+                         scale, key_chunk, chunk=0, window=0, keep_first=0, softcap=0.0, zero_sink=False, talk=None, max_context=0):
         group = heads // kv_heads
         for r in range(q.shape[0]):
             seg = int(row_seg[r])
@@ -616,27 +616,20 @@ class ReferenceOps:
             k = k_pages[pages, :, :, offs, :].double().reshape(len(keys), kv_heads, k_dim)
             v = v_pages[pages, :, :, offs].double()
             qr = q[r].double().view(heads, k_dim)
+            weights = []
             for h in range(heads):
                 s = (k[:, h // group, :] @ qr[h]) * scale
                 if softcap:
                     s = softcap * torch.tanh(s / softcap)
                 if zero_sink:
-                    p = torch.softmax(torch.cat([s, torch.zeros(1, dtype=s.dtype)]), dim=0)[:-1]
+                    weights.append(torch.softmax(torch.cat([s, torch.zeros(1, dtype=s.dtype)]), dim=0)[:-1])
                 else:
-                    p = torch.softmax(s, dim=0)
-                if spread:                     # this head's weights on the values of every key/value head
-                    n = kv_heads * v_dim
-                    out[r, h * n:(h + 1) * n] = torch.einsum("n,ngd->gd", p, v).reshape(-1).to(out.dtype)
-                else:
-                    out[r, h * v_dim:(h + 1) * v_dim] = (p @ v[:, h // group, :]).to(out.dtype)
-        return out
-
-    def mix_heads(self, spread, talk, out, heads, kv_heads, v_dim):
-        rows = spread.shape[0]
-        a = spread.double().view(rows, heads, kv_heads, v_dim)
-        group = heads // kv_heads
-        for h in range(heads):
-            out[:, h * v_dim:(h + 1) * v_dim] = torch.einsum("g,rgd->rd", talk[h].double(), a[:, :, h // group]).to(out.dtype)
+                    weights.append(torch.softmax(s, dim=0))
+            weights = torch.stack(weights)
+            if talk is not None:
+                weights = talk.double() @ weights
+            for h in range(heads):
+                out[r, h * v_dim:(h + 1) * v_dim] = (weights[h] @ v[:, h // group, :]).to(out.dtype)
         return out
 
     def gated_linear_attention(self, qkv, z, bias, tau, query_scale, state, row_seg, seg_start, slots, out, heads, dim, vdim, form="auto"):
