@@ -290,6 +290,27 @@ def dumizen_config(size, layers):
     return cfg, layers
 
 
+def zoguzen_config(size, layers):
+    """`layers` layers in turn: attention over the row's chunk with capped scores, a zero sink and mixed heads, one more that reads its
+    keys and values, minGRU of as many lanes as the heads have, and a pair of windowed attention (1,024 tokens and the first 64, an
+    output gate) beside gated linear attention (as many heads of the same size); convolutions of four taps; routed feed-forwards
+    everywhere, two of eight gated experts of half the dense width (a token multiplies as many weights as the dense layer has);
+    128 numbers a token and layer beside the stream."""
+    heads, kv_heads, dim, ff = size["heads"], size["kv_heads"], size["dim"], size["ff"]
+    base = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "conv": 4}
+    chunked = dict(base, softcap=50.0, mask={"size": DESIGN_CHUNK})
+    both = {"left": dict(base, mask={"size": 1024, "keep_first": 64},
+                         rot={"dims": dim, "base": 500000.0, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}),
+            "right": {"heads": heads, "dim": dim, "vdim": dim, "tau": 16.0}}
+    mlp = {"kind": "moe", "expert": {"ff": ff // DESIGN_TOP}, "router": {"experts": DESIGN_EXPERTS, "top": DESIGN_TOP}}
+    kinds = [lambda i: ("attention", chunked), lambda i: ("attention", dict(chunked, kv_from=i - 1)),
+             lambda i: ("mingru", {"width": heads * dim}), lambda i: ("parallel", both)]
+    made = [kinds[i % 4](i) for i in range(layers)]
+    cfg = {"architecture": "Zoguzen", "width": size["width"], "vocab": size["vocab"], "norm": {"eps": 1e-6}, "max_position": 32768,
+           "logit_softcap": 30.0, "token_side": {"dim": 128}, "layers": [{"type": t, "mixer": m, "mlp": mlp} for t, m in made]}
+    return cfg, layers
+
+
 def llama_config_of(size, layer_runs):
     return {"model_type": "llama", "architectures": ["LlamaForCausalLM"], "num_hidden_layers": layer_runs,
             "hidden_size": size["width"], "num_attention_heads": size["heads"], "num_key_value_heads": size["kv_heads"],
@@ -298,7 +319,7 @@ def llama_config_of(size, layer_runs):
 
 
 def design_run(args):
-    """Prefill and decode throughput of another design (Menitar, Purivik, Venadra, Dumizen) beside Llama at equal sizes (width, heads, head
+    """Prefill and decode throughput of another design (Menitar, Purivik, Venadra, Dumizen, Zoguzen) beside Llama at equal sizes (width, heads, head
     size, feed-forward, vocabulary, as many layers as the other has layer runs), random bfloat16 weights, with the device
     time of the kernels of a decode step and of a prefill step of each.  Prints one JSON line of its own."""
     import gc
@@ -308,10 +329,12 @@ def design_run(args):
     size = DESIGN_SIZES[args.design_size]
     layers = args.layers or size["layers"]
     design, layer_runs = {"menitar": menitar_config, "purivik": purivik_config, "venadra": venadra_config,
-                          "dumizen": dumizen_config}[args.design](size, layers)
+                          "dumizen": dumizen_config, "zoguzen": zoguzen_config}[args.design](size, layers)
     models = {args.design: (design, size["vocab"])}
     if args.design == "dumizen":       # its closest relative (norms behind the parts, routed experts, looped layers) stands beside it too
         models["purivik"] = (purivik_config(size, layers)[0], size["vocab"])
+    if args.design == "zoguzen":       # its closest relative (windowed attention, pairs, routed experts), every layer once
+        models["dumizen"] = ({k: v for k, v in dumizen_config(size, layers)[0].items() if k != "loop"}, size["vocab"])
     models["llama"] = (llama_config_of(size, layer_runs), size["vocab"])
     batches = sorted({1, args.batch, 64})
     steps, warmup = min(args.steps, 96), args.warmup
@@ -353,7 +376,7 @@ def design_run(args):
         print(f"[bench] {name} prefill {PREFILL_TOKENS} tokens: {best * 1e3:.2f} ms", file=sys.stderr, flush=True)
         if not args.no_kernels:
             out["kernels"] = {}
-            found = kernel_breakdown(one_prompt, 2, top=12)
+            found = kernel_breakdown(one_prompt, 2, top=24 if args.design == "zoguzen" else 12)
             if found:
                 out["kernels"]["prefill_us"] = found
             names = [f"{name}-k{i}" for i in range(args.batch)]
@@ -363,7 +386,7 @@ def design_run(args):
             while min(got.values()) < 4:
                 for ev in engine.step():
                     got[ev.request_id] += 1
-            found = kernel_breakdown(engine.step, 5, top=12)
+            found = kernel_breakdown(engine.step, 5, top=24 if args.design == "zoguzen" else 12)
             if found:
                 out["kernels"][f"decode_b{args.batch}_us"] = found
             for n in names:
@@ -412,7 +435,7 @@ def main():
     ap.add_argument("--sampled", action="store_true",
                     help="for profiling the sampling kernels: the decode runs draw with temperature 0.8, top-k 50 and top-p 0.9 under a "
                          "repetition penalty of 1.1 and report 5 log-probabilities a token (the headline run is greedy)")
-    ap.add_argument("--design", choices=["menitar", "purivik", "venadra", "dumizen"], default=None,
+    ap.add_argument("--design", choices=["menitar", "purivik", "venadra", "dumizen", "zoguzen"], default=None,
                     help="instead of the headline run: prefill and decode of this design beside Llama at equal sizes, with the kernels' "
                          "device times of both; prints a line of its own")
     ap.add_argument("--design-size", choices=sorted(DESIGN_SIZES), default="1.5b", help="with --design: the layer sizes")
