@@ -22,6 +22,7 @@ namespace {
 constexpr int kThreads = 256;
 constexpr int kWavesM = kThreads / kWave;
 constexpr float kLog2e = 1.4426950408889634f;
+constexpr float kFixedCap = 90.f;      // caps, in units of log2, up to which exponentials are taken without a running maximum
 
 struct MaskedParams {
     const bf16_t *q;
@@ -61,13 +62,16 @@ __device__ __forceinline__ float weigh8(const float (&s)[8], float m_new, bf16x8
     float sum = 0.f;
 #pragma unroll
     for (int e = 0; e < 8; e++) {
-        const float w = s[e] == -INFINITY ? 0.f : fast_exp2(s[e] - m_new);
+        const float w = fast_exp2(s[e] - m_new);      // 0 for keys that are not seen: m_new is a number
         sum += w;
         hi[e] = (bf16_t)w;
         lo[e] = (bf16_t)(w - (float)hi[e]);
     }
     return sum;
 }
+
+// where key (0 .. 63) of a tile stands in LDS: the sixteen keys of a product's A rows one behind the other
+__device__ __forceinline__ int key_row(int key) { return (key & 32) | ((key & 4) << 2) | ((key & 24) >> 1) | (key & 3); }
 
 __device__ __forceinline__ bf16x8_t zero8() {
     bf16x8_t z;
@@ -141,26 +145,44 @@ masked_rows_kernel(const MaskedParams p) {
     const int tiles = first_tiles + (pos_last - main0) / KT + 1;
     const int cps = psh < 6 ? psh - 3 : 3;       // log2 of the 8-token pieces of a value lane that lie together in a page and tile
 
+    // A tile's pages are looked up two tiles ahead and its keys and values asked for one tile ahead, so that neither is waited for:
+    // a thread's K pieces are of one key, its V pieces of VCH stretches of tokens.
     bf16x8_t rk[KCH], rv[VCH];
+    int page_k, page_v[VCH];
     auto tile_base = [&](int t) { return t < first_tiles ? t * KT : main0 + (t - first_tiles) * KT; };
+    auto v_place = [&](int i, int &nv, int &d, int &koff) {
+        const int ch = threadIdx.x + i * kThreads;
+        nv = ch / (DV * KT / 8);
+        const int r0 = ch - nv * (DV * KT / 8);
+        const int pg = r0 / (DV << cps), r1 = r0 - pg * (DV << cps);       // stretches of 8 << cps tokens
+        d = r1 >> cps, koff = (pg << (cps + 3)) + (r1 & ((1 << cps) - 1)) * 8;
+    };
+    auto look_up = [&](int t) {
+        const int k0 = tile_base(t);
+        page_k = tbl[min(k0 + (int)(threadIdx.x & (KT - 1)), pos_last) >> psh];
+#pragma unroll
+        for (int i = 0; i < VCH; i++) {
+            int nv, d, koff;
+            v_place(i, nv, d, koff);
+            page_v[i] = tbl[min(k0 + koff, pos_last) >> psh];
+        }
+    };
     auto issue = [&](int t) {
         const int k0 = tile_base(t);
+        {
+            const int kabs = min(k0 + (int)(threadIdx.x & (KT - 1)), pos_last);      // keys behind the tile's last row: an address that exists; masked
+            const bf16_t *kr = p.k_pages + key_offset(page_k, p.kv_heads, kvh, ps, D, kabs & pmask, threadIdx.x / KT * 8);
 #pragma unroll
-        for (int i = 0; i < KCH; i++) {
-            const int ch = threadIdx.x + i * kThreads, key = ch & (KT - 1), dc = ch / KT;
-            const int kabs = min(k0 + key, pos_last);      // keys behind the tile's last row: an address that exists; masked
-            rk[i] = *(const bf16x8_t *)(p.k_pages + key_offset(tbl[kabs >> psh], p.kv_heads, kvh, ps, D, kabs & pmask, dc * 8));
+            for (int i = 0; i < KCH; i++) rk[i] = *(const bf16x8_t *)(kr + (size_t)i * (kThreads / KT) * ps * 8);
         }
 #pragma unroll
         for (int i = 0; i < VCH; i++) {
-            const int ch = threadIdx.x + i * kThreads;
-            const int nv = ch / (DV * KT / 8), r0 = ch - nv * (DV * KT / 8);
-            const int pg = r0 / (DV << cps), r1 = r0 - pg * (DV << cps);       // stretches of 8 << cps tokens
-            const int d = r1 >> cps, koff = (pg << (cps + 3)) + (r1 & ((1 << cps) - 1)) * 8;
+            int nv, d, koff;
+            v_place(i, nv, d, koff);
             const int kabs = k0 + koff;
             bf16x8_t v = zero8();
             if (kabs <= pos_last) {
-                v = *(const bf16x8_t *)(p.v_pages + (((size_t)tbl[kabs >> psh] * p.kv_heads + vh0 + nv) * DV + d) * ps + (kabs & pmask));
+                v = *(const bf16x8_t *)(p.v_pages + (((size_t)page_v[i] * p.kv_heads + vh0 + nv) * DV + d) * ps + (kabs & pmask));
                 if (kabs + 7 > pos_last)      // slots past the last token hold whatever an earlier request left
 #pragma unroll
                     for (int e = 0; e < 8; e++)
@@ -173,14 +195,12 @@ masked_rows_kernel(const MaskedParams p) {
 #pragma unroll
         for (int i = 0; i < KCH; i++) {
             const int ch = threadIdx.x + i * kThreads;
-            *(bf16x8_t *)(Ks + (ch & (KT - 1)) * KP + ch / KT * 8) = rk[i];
+            *(bf16x8_t *)(Ks + key_row(ch & (KT - 1)) * KP + ch / KT * 8) = rk[i];
         }
 #pragma unroll
         for (int i = 0; i < VCH; i++) {
-            const int ch = threadIdx.x + i * kThreads;
-            const int nv = ch / (DV * KT / 8), r0 = ch - nv * (DV * KT / 8);
-            const int pg = r0 / (DV << cps), r1 = r0 - pg * (DV << cps);
-            const int d = r1 >> cps, koff = (pg << (cps + 3)) + (r1 & ((1 << cps) - 1)) * 8;
+            int nv, d, koff;
+            v_place(i, nv, d, koff);
             *(bf16x8_t *)(Vs + (nv * DV + d) * VP + koff) = rv[i];
         }
     };
@@ -189,11 +209,19 @@ masked_rows_kernel(const MaskedParams p) {
 #pragma unroll
     for (int t = 0; t < NV * VT; t++) o[t] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
     float m_run = -INFINITY, l_run = 0.f;
+    look_up(0);
     issue(0);
+    if (tiles > 1) look_up(1);
+    // Capped scores lie within the cap: their exponentials need no reference of their own, and nothing is ever rescaled (exp2 of up to
+    // kFixedCap either way leaves a float room for any number of keys).
+    const bool fixed = p.cap_log2 > 0.f && p.cap_log2 <= kFixedCap;
+    if (fixed) m_run = 0.f;
+    const int lo_last = range_start(p, pos_last);
     for (int t = 0; t < tiles; t++) {
         __syncthreads();      // the tile before has been read
         commit();
         if (t + 1 < tiles) issue(t + 1);
+        if (t + 2 < tiles) look_up(t + 2);
         __syncthreads();
         const int k0 = tile_base(t);
         const bool firsts = t < first_tiles;
@@ -201,29 +229,40 @@ masked_rows_kernel(const MaskedParams p) {
 #pragma unroll
         for (int i = 0; i < 4; i++) {
             st[i] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
-            const int key_local = (i >> 1) * 32 + (c >> 2) * 8 + (i & 1) * 4 + (c & 3);
 #pragma unroll
             for (int kk = 0; kk < KD; kk++) {
-                const bf16x8_t a = *(const bf16x8_t *)(Ks + key_local * KP + kk * 32 + g * 8);
+                const bf16x8_t a = *(const bf16x8_t *)(Ks + (i * 16 + c) * KP + kk * 32 + g * 8);
                 st[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, qf[kk], st[i], 0, 0, 0);
             }
         }
         float s[2][8];
         float m_blk = -INFINITY;
+        // a tile that every row of the workgroup sees whole needs no mask (the queries of no row compute what is dropped)
+        const bool whole = firsts ? k0 + KT <= first_end : k0 >= lo_last && k0 + KT - 1 <= pos0;
 #pragma unroll
         for (int b = 0; b < 2; b++)
 #pragma unroll
-            for (int e = 0; e < 8; e++) {
-                const int key = k0 + b * 32 + g * 8 + e;
-                const bool vis = key <= my_pos && (firsts ? key < p.keep_first && key < my_lo : key >= my_lo || key < p.keep_first) &&
-                                 (!firsts || key < first_end);
-                s[b][e] = vis ? score_of(p, st[b * 2 + (e >> 2)][e & 3]) : -INFINITY;
-                m_blk = fmaxf(m_blk, s[b][e]);
-            }
-        m_blk = fmaxf(m_blk, __shfl_xor(m_blk, 16, kWave));
-        m_blk = fmaxf(m_blk, __shfl_xor(m_blk, 32, kWave));
-        const float m_new = fmaxf(m_run, m_blk);
-        if (__any(m_new > m_run)) {      // the outputs are rescaled only when some row's maximum moved
+            for (int e = 0; e < 8; e++) s[b][e] = score_of(p, st[b * 2 + (e >> 2)][e & 3]);
+        if (!whole)
+#pragma unroll
+            for (int b = 0; b < 2; b++)
+#pragma unroll
+                for (int e = 0; e < 8; e++) {
+                    const int key = k0 + b * 32 + g * 8 + e;
+                    const bool vis = key <= my_pos && (firsts ? key < first_end : key >= my_lo || key < p.keep_first);
+                    s[b][e] = vis ? s[b][e] : -INFINITY;
+                }
+        float m_new = m_run;
+        if (!fixed) {
+#pragma unroll
+            for (int b = 0; b < 2; b++)
+#pragma unroll
+                for (int e = 0; e < 8; e++) m_blk = fmaxf(m_blk, s[b][e]);
+            m_blk = fmaxf(m_blk, __shfl_xor(m_blk, 16, kWave));
+            m_blk = fmaxf(m_blk, __shfl_xor(m_blk, 32, kWave));
+            m_new = fmaxf(m_run, m_blk);
+        }
+        if (!fixed && __any(m_new > m_run)) {      // the outputs are rescaled only when some row's maximum moved
             const float alpha = m_run == -INFINITY ? 0.f : fast_exp2(m_run - m_new);
             l_run *= alpha;
 #pragma unroll
@@ -233,7 +272,7 @@ masked_rows_kernel(const MaskedParams p) {
 #pragma unroll
         for (int b = 0; b < 2; b++) {
             bf16x8_t hi, lo;
-            l_run += weigh8(s[b], m_run, hi, lo);
+            l_run += weigh8(s[b], m_run == -INFINITY ? 0.f : m_run, hi, lo);
 #pragma unroll
             for (int i = 0; i < NV * VT; i++) {
                 const bf16x8_t a = *(const bf16x8_t *)(Vs + (i * 16 + c) * VP + b * 32 + g * 8);
@@ -336,8 +375,7 @@ masked_heads_kernel(const MaskedParams p) {
         const float m_new = fmaxf(m_run, m_blk);
         const float alpha = m_run == -INFINITY ? 0.f : fast_exp2(m_run - m_new);
         bf16x8_t hi, lo8;
-        l_run = l_run * alpha + (m_new == -INFINITY ? 0.f : weigh8(s, m_new, hi, lo8));
-        if (m_new == -INFINITY) hi = lo8 = zero8();
+        l_run = l_run * alpha + weigh8(s, m_new == -INFINITY ? 0.f : m_new, hi, lo8);
         m_run = m_new;
 #pragma unroll
         for (int t = 0; t < NV * VT; t++) {
@@ -375,22 +413,26 @@ masked_heads_kernel(const MaskedParams p) {
     }
 }
 
-// The shares put together in their order: grid (rows, key/value heads of the outputs).  Without `talk` the workgroup writes its key/value
-// head's outputs; with it, it gathers what every head's weights made of this key/value head's values and mixes: out_h = sum_g
-// talk[h][g] A_g.  LDS: heads * DV floats and a factor a head and split.
+// The shares put together in their order: grid (rows, key/value heads of the outputs, slices of value lanes).  Without `talk` the
+// workgroup writes its key/value head's outputs; with it, it gathers what every head's weights made of this key/value head's values
+// and mixes: out_h = sum_g talk[h][g] A_g.
 __global__ void __launch_bounds__(kThreads)
 masked_merge_kernel(const float *__restrict__ parts, int splits, const int32_t *__restrict__ row_seg, const float *__restrict__ talk,
-                    bf16_t *__restrict__ out, int heads, int kv_heads, int DV, int NV, int zero_sink) {
+                    bf16_t *__restrict__ out, int heads, int kv_heads, int DV, int NV, int zero_sink, int lanes) {
     extern __shared__ float smem[];
     const int row = blockIdx.x, vh = blockIdx.y, G = heads / kv_heads;
     bf16_t *dst = out + ((size_t)row * heads + vh * G) * DV;
     if (row_seg[row] < 0) {      // padding row: zeros
-        for (int i = threadIdx.x; i < G * DV; i += kThreads) dst[i] = (bf16_t)0.f;
+        if (blockIdx.z == 0)
+            for (int i = threadIdx.x; i < G * DV; i += kThreads) dst[i] = (bf16_t)0.f;
         return;
     }
     const int count = talk != nullptr ? heads : G, first = talk != nullptr ? 0 : vh * G;      // heads whose shares this workgroup reads
-    float *factor = smem;                       // [count][splits]
-    float *A = factor + count * splits;         // [count][DV]
+    // blockIdx.z: a slice of `lanes` value lanes
+    float *factor = smem;                       // [count][splits]: the shares' maxima, then their factors
+    float *denom = factor + count * splits;     // [count][splits]
+    float *A = denom + count * splits;          // [count][lanes]
+    const int d0 = blockIdx.z * lanes;
     const int W = NV * DV, stride = 16 * W + 32;
     const int groups = talk != nullptr ? kv_heads / NV : 1, at = talk != nullptr ? vh % NV : 0;
     const int ny = kv_heads * groups, yv = talk != nullptr ? vh / NV : 0;
@@ -398,14 +440,18 @@ masked_merge_kernel(const float *__restrict__ parts, int splits, const int32_t *
         const int kvh = h / G;
         return parts + (((size_t)row * ny + yv * kv_heads + kvh) * splits + s) * stride;
     };
+    for (int i = threadIdx.x; i < count * splits; i += kThreads) {
+        const int h = first + i / splits, s = i % splits, q = h % G;
+        factor[i] = share(h, s)[16 * W + q];
+        denom[i] = share(h, s)[16 * W + 16 + q];
+    }
+    __syncthreads();
     for (int i = threadIdx.x; i < count; i += kThreads) {
-        const int h = first + i, q = h % G;
         float m = -INFINITY, l = 0.f;
-        for (int s = 0; s < splits; s++) m = fmaxf(m, share(h, s)[16 * W + q]);
+        for (int s = 0; s < splits; s++) m = fmaxf(m, factor[i * splits + s]);
         for (int s = 0; s < splits; s++) {
-            const float ms = share(h, s)[16 * W + q];
-            const float f = ms == -INFINITY ? 0.f : fast_exp2(ms - m);
-            l += share(h, s)[16 * W + 16 + q] * f;
+            const float ms = factor[i * splits + s], f = ms == -INFINITY ? 0.f : fast_exp2(ms - m);
+            l += denom[i * splits + s] * f;
             factor[i * splits + s] = f;
         }
         if (zero_sink) l += fast_exp2(-m);
@@ -413,22 +459,23 @@ masked_merge_kernel(const float *__restrict__ parts, int splits, const int32_t *
         for (int s = 0; s < splits; s++) factor[i * splits + s] *= inv;
     }
     __syncthreads();
-    for (int idx = threadIdx.x; idx < count * DV; idx += kThreads) {
-        const int i = idx / DV, d = idx - i * DV, h = first + i, q = h % G;
+    for (int idx = threadIdx.x; idx < count * lanes; idx += kThreads) {
+        const int i = idx / lanes, d = idx - i * lanes, h = first + i, q = h % G;
         float acc = 0.f;
-#pragma unroll 4
-        for (int s = 0; s < splits; s++) acc = fmaf(share(h, s)[q * W + at * DV + d], factor[i * splits + s], acc);
-        if (talk == nullptr) dst[idx] = (bf16_t)acc;
+#pragma unroll 8
+        for (int s = 0; s < splits; s++) acc = fmaf(share(h, s)[q * W + at * DV + d0 + d], factor[i * splits + s], acc);
+        if (talk == nullptr) dst[i * DV + d0 + d] = (bf16_t)acc;
         else A[idx] = acc;
     }
     if (talk == nullptr) return;
     __syncthreads();
-    for (int idx = threadIdx.x; idx < G * DV; idx += kThreads) {
-        const int hl = idx / DV, d = idx - hl * DV;
+    for (int idx = threadIdx.x; idx < G * lanes; idx += kThreads) {
+        const int hl = idx / lanes, d = idx - hl * lanes;
         const float *tk = talk + (size_t)(vh * G + hl) * heads;
         float acc = 0.f;
-        for (int g = 0; g < heads; g++) acc = fmaf(tk[g], A[g * DV + d], acc);
-        dst[idx] = (bf16_t)acc;
+#pragma unroll 4
+        for (int g = 0; g < heads; g++) acc = fmaf(tk[g], A[g * lanes + d], acc);
+        dst[hl * DV + d0 + d] = (bf16_t)acc;
     }
 }
 
@@ -493,8 +540,7 @@ int fllm_masked_attention_bf16_fast(const void *q, int q_stride, const void *k_p
         const size_t room = (bytes - kWorkspaceCounterBytes) / sizeof(float), each = (size_t)tiles * (16 * NV * v_dim + 32);
         splits = std::min<long>(splits, (long)(room / each));
         if (splits < 1) return 1;
-        const size_t smem = (size_t)(talk != nullptr ? heads : G) * (splits + v_dim) * sizeof(float);
-        if (smem > 64 * 1024) return 1;
+        if ((size_t)(talk != nullptr ? heads : G) * (2 * splits + 32) * sizeof(float) > 64 * 1024) return 1;      // what the merge keeps in LDS
         p.splits = (int)splits;
         p.parts = (float *)((char *)base + kWorkspaceCounterBytes);
         grid = dim3(rows, kv_heads * groups, (unsigned)splits);
@@ -518,9 +564,10 @@ int fllm_masked_attention_bf16_fast(const void *q, int q_stride, const void *k_p
 #undef FLLM_KD
     *mixed = 0;
     if (by_heads) {
-        const size_t smem = (size_t)(talk != nullptr ? heads : G) * (p.splits + v_dim) * sizeof(float);
-        hipLaunchKernelGGL(masked_merge_kernel, dim3(rows, kv_heads), dim3(kThreads), smem, stream, p.parts, p.splits, row_seg, talk, (bf16_t *)out,
-                           heads, kv_heads, v_dim, NV, zero_sink);
+        const int lanes = 32;      // value lanes a workgroup of the merge: v_dim is a multiple
+        const size_t smem = (size_t)(talk != nullptr ? heads : G) * (2 * p.splits + lanes) * sizeof(float);
+        hipLaunchKernelGGL(masked_merge_kernel, dim3(rows, kv_heads, v_dim / lanes), dim3(kThreads), smem, stream, p.parts, p.splits, row_seg, talk,
+                           (bf16_t *)out, heads, kv_heads, v_dim, NV, zero_sink, lanes);
         *mixed = 1;
     }
     return fllm_check_launch("masked_attention (matrix cores)");

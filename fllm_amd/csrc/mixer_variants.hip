@@ -491,20 +491,29 @@ masked_attention_kernel(const T *__restrict__ q, int q_stride, const T *__restri
 }
 
 // spread [row][head][value head][v_dim] float32 -> out[row][head][v_dim]: out_h = sum_g talk[h][g] spread[g][value head of h].
-// grid (rows, blocks of outputs); the sum runs in head order.
-template <typename T>
+// grid (rows, blocks of outputs); the sum runs in head order.  V: neighbouring lanes a thread (4 where v_dim is a multiple).
+template <typename T, int V>
 __global__ void __launch_bounds__(kBlock)
 mix_heads_kernel(const float *__restrict__ spread, const float *__restrict__ talk, T *__restrict__ out, int heads, int kv_heads, int v_dim) {
     const size_t r = blockIdx.x;
-    const int o = blockIdx.y * kBlock + threadIdx.x;
+    const int o = (blockIdx.y * kBlock + threadIdx.x) * V;
     if (o >= heads * v_dim) return;
     const int h = o / v_dim, c = o - h * v_dim, vh = h / (heads / kv_heads);
     const float *src = spread + (r * heads * kv_heads + vh) * v_dim + c;
     const float *tk = talk + (size_t)h * heads;
-    float acc = 0.f;
+    float acc[V];
+#pragma unroll
+    for (int e = 0; e < V; e++) acc[e] = 0.f;
 #pragma unroll 8
-    for (int g = 0; g < heads; g++) acc = fmaf(tk[g], src[(size_t)g * kv_heads * v_dim], acc);
-    out[r * heads * v_dim + o] = from_f32<T>(acc);
+    for (int g = 0; g < heads; g++) {
+        float a[V];
+        if constexpr (V == 4) *(f32x4_t *)a = *(const f32x4_t *)(src + (size_t)g * kv_heads * v_dim);
+        else a[0] = src[(size_t)g * kv_heads * v_dim];
+#pragma unroll
+        for (int e = 0; e < V; e++) acc[e] = fmaf(tk[g], a[e], acc[e]);
+    }
+#pragma unroll
+    for (int e = 0; e < V; e++) out[r * heads * v_dim + o + e] = from_f32<T>(acc[e]);
 }
 
 // ---- operands of a linear attention: rotated, scaled, float32 ----------------------------------------------------------------
@@ -752,13 +761,18 @@ extern "C" int fllm_masked_attention(const void *q, int q_stride, const void *k_
     FLLM_REQUIRE(q && k_pages && v_pages && tables && row_pos && row_seg && out, "masked_attention: operands missing");
     FLLM_REQUIRE(talk == nullptr || spread != nullptr, "masked_attention: heads that are mixed need room for their spread values");
     if (rows == 0) return 0;
-    const dim3 mix_grid(rows, (heads * v_dim + kBlock - 1) / kBlock);
+    const int mix_lanes = v_dim % 4 == 0 ? 4 : 1;
+    const dim3 mix_grid(rows, (heads * v_dim / mix_lanes + kBlock - 1) / kBlock);
     FLLM_REQUIRE(mix_grid.y <= 65535, "masked_attention: too many heads");
     auto mix = [&]() {
-        if (dtype == FLLM_F32)
-            hipLaunchKernelGGL(mix_heads_kernel<float>, mix_grid, dim3(kBlock), 0, stream, spread, talk, (float *)out, heads, kv_heads, v_dim);
+        if (dtype == FLLM_F32 && mix_lanes == 4)
+            hipLaunchKernelGGL((mix_heads_kernel<float, 4>), mix_grid, dim3(kBlock), 0, stream, spread, talk, (float *)out, heads, kv_heads, v_dim);
+        else if (dtype == FLLM_F32)
+            hipLaunchKernelGGL((mix_heads_kernel<float, 1>), mix_grid, dim3(kBlock), 0, stream, spread, talk, (float *)out, heads, kv_heads, v_dim);
+        else if (mix_lanes == 4)
+            hipLaunchKernelGGL((mix_heads_kernel<bf16_t, 4>), mix_grid, dim3(kBlock), 0, stream, spread, talk, (bf16_t *)out, heads, kv_heads, v_dim);
         else
-            hipLaunchKernelGGL(mix_heads_kernel<bf16_t>, mix_grid, dim3(kBlock), 0, stream, spread, talk, (bf16_t *)out, heads, kv_heads, v_dim);
+            hipLaunchKernelGGL((mix_heads_kernel<bf16_t, 1>), mix_grid, dim3(kBlock), 0, stream, spread, talk, (bf16_t *)out, heads, kv_heads, v_dim);
     };
     if (dtype == FLLM_BF16 && key_chunk == 8) {
         int mixed = 0;
