@@ -321,7 +321,7 @@ int fllm_experts_down(const void *act, const int32_t *ids, int pairs, const void
                       hipStream_t stream);
 // The same products on the matrix cores (bfloat16): the pairs are grouped by expert on the device and multiplied as tiles of
 // 64 or 128 rows.  0: launched; 1: shape declined (the caller runs the plain kernels).  act and xs: scratch, bfloat16
-// [rows * top, inter] and [rows * top, K]; out: float32 [rows * top, N]; work: fllm_experts_grouped_work_ints(rows * top, E)
+// [rows * top, inter] and [rows * top, K] (weights null: all 1, and no xs); out: float32 [rows * top, N]; work: fllm_experts_grouped_work_ints(rows * top, E)
 // int32 of scratch.
 size_t fllm_experts_grouped_work_ints(int pairs, int E);
 size_t fllm_experts_grouped_plane_floats(int pairs, int E, int N, int inter);   // `planes`: float32 scratch of that many (0: none)
@@ -444,6 +444,11 @@ int fllm_experts_grouped_ungated(const void *h, int ldh, const int32_t *ids, int
 // out1[i] = (x[r] - mean) * rsqrt(mean (x[r] - mean)^2 + eps1) * w1, r = rows ? rows[i] : i, and with w2 the same with w2 and eps2 in out2.
 int fllm_layernorm(const float *x, const int32_t *rows, const float *w1, float eps1, void *out1, const float *w2, float eps2, void *out2,
                    int count, int width, int out_dtype, hipStream_t stream);
+// fllm_layernorm of both weights (w2 may be null), the first norm's values (rounded to out_dtype) through fllm_short_conv on their way to
+// out1, for steps of one row a segment (segment s is row s); rows of at most 8192 values.
+int fllm_layernorm_conv(const float *x, const float *w1, float eps1, const float *conv, int taps, void *state, const int32_t *row_seg,
+                        const int32_t *slots, void *out1, const float *w2, float eps2, void *out2, int rows, int width, int out_dtype,
+                        hipStream_t stream);
 // out = a x / rms(x) wx + b y / rms(y) wy over rows of `width` (accumulate: out += ..), float32.
 int fllm_normed_pair_sum(float *out, const float *x, const float *wx, float a, const float *y, const float *wy, float b, float eps, int rows,
                          int width, int accumulate, hipStream_t stream);
@@ -454,6 +459,10 @@ int fllm_softcap(float *x, size_t total, float cap, hipStream_t stream);
 // out[r, c] = gelu_tanh(z[r, c]) * table[ids[r], offset + c], rows of `dim`; table [vocab, table_width] of `dtype`.
 int fllm_gelu_side(const void *z, const int32_t *ids, const void *table, int vocab, int table_width, int offset, void *out, int rows, int dim,
                    int dtype, hipStream_t stream);
+// The same of z = W x (x float32 [rows, width], rounded to `dtype` first; W [dim, width]) in one kernel.  1: declined (more than 8 rows, a
+// width that is no multiple of 8).
+int fllm_side_gate(const float *x, const void *w, const int32_t *ids, const void *table, int vocab, int table_width, int offset, void *out,
+                   int rows, int width, int dim, int dtype, hipStream_t stream);
 
 // ---- projections behind a short convolution (conv_store.hip) ----
 // Rows [q | k | v | ..] of `ld` elements (store_kv 0: q alone passes the convolution).  Channel c of the row at position p: y = sum_j

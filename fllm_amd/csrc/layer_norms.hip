@@ -3,9 +3,11 @@
 //
 //   layernorm         out = (x - mean) * rsqrt(mean (x - mean)^2 + eps) * w, of every row or of the rows named; with a second
 //                     weight vector (and eps) both norms of a row in one pass.
+//   layernorm_conv    the same for steps of one row a segment, the first norm through a short convolution over time on its way.
 //   normed_pair_sum   out (+)= a x / rms(x) wx + b y / rms(y) wy.
 //   cast_rows, softcap, gelu_side: a stream's rows in the compute type; cap * tanh(x / cap); gelu(z) times a part of the rows'
 //                     tokens' rows in a table.
+//   side_gate         gelu_side of z = W x in one kernel, for steps of few rows.
 #include "api.h"
 #include "common.h"
 
@@ -13,6 +15,7 @@ namespace {
 
 constexpr int kBlock = 256;
 constexpr int kWaves = kBlock / kWave;
+constexpr int kMaxKeep = 15;
 
 // N > 0: the row (at most N * kBlock values) stays in registers between the mean, the deviations and the output; 0: any width
 template <typename T, int N>
@@ -67,6 +70,67 @@ layernorm_kernel(const float *__restrict__ x, const int32_t *__restrict__ rows, 
     }
 }
 
+// grid (rows, blocks of kBlock channels): every workgroup of a row sums the row itself, in layernorm_kernel's order, so that no
+// thread loops over channels behind the sums and all it reads is on its way at once.  The first norm's value is rounded to T before
+// the convolution, as layernorm_kernel's output is.  A thread owns a channel of the state: it reads the old entries before it
+// writes any.
+template <typename T, int N>
+__global__ void __launch_bounds__(kBlock)
+layernorm_conv_kernel(const float *__restrict__ x, const float *__restrict__ w1, float eps1, const float *__restrict__ conv, int taps,
+                      T *__restrict__ state, const int32_t *__restrict__ row_seg, const int32_t *__restrict__ slots, T *__restrict__ out1,
+                      const float *__restrict__ w2, float eps2, T *__restrict__ out2, int width) {
+    __shared__ float scratch[kWaves];
+    const int r = blockIdx.x, c = blockIdx.y * kBlock + threadIdx.x;
+    const bool mine = c < width;
+    T *d1 = out1 + (size_t)r * width, *d2 = out2 == nullptr ? nullptr : out2 + (size_t)r * width;
+    const int seg = row_seg[r];
+    if (seg < 0) {      // padding row
+        if (mine) d1[c] = from_f32<T>(0.f);
+        if (mine && d2 != nullptr) d2[c] = from_f32<T>(0.f);
+        return;
+    }
+    const int keep = taps - 1;
+    T *old = state + (size_t)slots[seg] * keep * width;
+    const float *wc = conv + (size_t)c * taps;
+    T held[kMaxKeep];
+#pragma unroll
+    for (int i = 0; i < kMaxKeep; i++)
+        if (i < keep && mine) held[i] = old[(size_t)i * width + c];
+    const float *src = x + (size_t)r * width;
+    const float own = mine ? src[c] : 0.f, a1 = mine ? w1[c] : 0.f, a2 = mine && d2 != nullptr ? w2[c] : 0.f;
+    float v[N];
+    float sum = 0.f;
+#pragma unroll
+    for (int j = 0; j < N; j++) {
+        const int at = threadIdx.x + j * kBlock;
+        v[j] = at < width ? src[at] : 0.f;
+        sum += v[j];
+    }
+    const float mean = block_sum<kWaves>(sum, scratch) / (float)width;
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < N; j++) {
+        v[j] -= mean;
+        if (threadIdx.x + j * kBlock < width) ss = fmaf(v[j], v[j], ss);
+    }
+    const float var = block_sum<kWaves>(ss, scratch) / (float)width;
+    if (!mine) return;
+    const float inv1 = 1.0f / sqrtf(var + eps1), inv2 = 1.0f / sqrtf(var + eps2);
+    const T h = from_f32<T>((own - mean) * (inv1 * a1));
+    const float now = to_f32<T>(h);
+    float acc = 0.f;
+#pragma unroll
+    for (int i = 0; i < kMaxKeep; i++) {      // oldest input first; entry i moves to i - 1
+        if (i >= keep) break;
+        acc = fmaf(wc[i], to_f32<T>(held[i]), acc);
+        if (i > 0) old[(size_t)(i - 1) * width + c] = held[i];
+    }
+    if (keep > 0) old[(size_t)(keep - 1) * width + c] = h;
+    acc = fmaf(wc[keep], now, acc);
+    d1[c] = from_f32<T>(now + acc);
+    if (d2 != nullptr) d2[c] = from_f32<T>((own - mean) * (inv2 * a2));
+}
+
 __global__ void __launch_bounds__(kBlock)
 normed_pair_sum_kernel(float *__restrict__ out, const float *__restrict__ x, const float *__restrict__ wx, float a, const float *__restrict__ y,
                        const float *__restrict__ wy, float b, float eps, int width, int accumulate) {
@@ -104,6 +168,17 @@ __device__ __forceinline__ float gelu_tanh(float z) {
     return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }
 
+__device__ __forceinline__ void load8(const float *p, float (&v)[8]) {
+    *(f32x4_t *)v = *(const f32x4_t *)p;
+    *(f32x4_t *)(v + 4) = *(const f32x4_t *)(p + 4);
+}
+
+__device__ __forceinline__ void load8(const bf16_t *p, float (&v)[8]) {
+    const bf16x8_t a = *(const bf16x8_t *)p;
+#pragma unroll
+    for (int e = 0; e < 8; e++) v[e] = (float)a[e];
+}
+
 template <typename T>
 __global__ void __launch_bounds__(kBlock)
 gelu_side_kernel(const T *__restrict__ z, const int32_t *__restrict__ ids, const T *__restrict__ table, int vocab, int table_width, int offset,
@@ -115,6 +190,51 @@ gelu_side_kernel(const T *__restrict__ z, const int32_t *__restrict__ ids, const
         id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);      // ids are validated on the host; never read outside the table
         out[i] = from_f32<T>(gelu_tanh(to_f32<T>(z[i])) * to_f32<T>(table[(size_t)id * table_width + offset + c]));
     }
+}
+
+// One workgroup an output lane d: z = W[d] . x for the R rows of the step (x rounded to T first, as cast_rows gives it), then
+// gelu_side of it.  dims that are multiples of 8 lie side by side in 16-byte loads.
+template <typename T, int R>
+__global__ void __launch_bounds__(kBlock)
+side_gate_kernel(const float *__restrict__ x, const T *__restrict__ w, const int32_t *__restrict__ ids, const T *__restrict__ table, int vocab,
+                 int table_width, int offset, T *__restrict__ out, int rows, int width, int dim) {
+    __shared__ float part[kWaves][R];
+    const int d = blockIdx.x, lane = threadIdx.x & (kWave - 1), wave = threadIdx.x / kWave;
+    const T *wr = w + (size_t)d * width;
+    float acc[R];
+#pragma unroll
+    for (int r = 0; r < R; r++) acc[r] = 0.f;
+    for (int c0 = threadIdx.x * 8; c0 < width; c0 += kBlock * 8) {
+        float wv[8];
+        load8(wr + c0, wv);
+#pragma unroll
+        for (int r = 0; r < R; r++) {
+            const float *xr = x + (size_t)(r < rows ? r : 0) * width + c0;
+            const f32x4_t a = *(const f32x4_t *)xr, b = *(const f32x4_t *)(xr + 4);
+#pragma unroll
+            for (int e = 0; e < 4; e++) acc[r] = fmaf(wv[e], to_f32<T>(from_f32<T>(a[e])), acc[r]);
+#pragma unroll
+            for (int e = 0; e < 4; e++) acc[r] = fmaf(wv[4 + e], to_f32<T>(from_f32<T>(b[e])), acc[r]);
+        }
+    }
+#pragma unroll
+    for (int r = 0; r < R; r++) {
+        acc[r] = wave_sum(acc[r]);
+        if (lane == 0) part[wave][r] = acc[r];
+    }
+    const int r = threadIdx.x;
+    float e = 0.f;
+    if (r < rows) {
+        int id = ids[r];
+        id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);      // ids are validated on the host; never read outside the table
+        e = to_f32<T>(table[(size_t)id * table_width + offset + d]);
+    }
+    __syncthreads();
+    if (r >= rows) return;
+    float z = 0.f;
+#pragma unroll
+    for (int w = 0; w < kWaves; w++) z += part[w][r];
+    out[(size_t)r * dim + d] = from_f32<T>(gelu_tanh(z) * e);
 }
 
 int small_grid(size_t total) {
@@ -144,6 +264,56 @@ extern "C" int fllm_layernorm(const float *x, const int32_t *rows, const float *
     else if (out_dtype == FLLM_BF16) launch_layernorm<bf16_t>(x, rows, w1, eps1, (bf16_t *)out1, w2, eps2, (bf16_t *)out2, count, width, stream);
     else FLLM_REQUIRE(false, "layernorm: unknown dtype %d", out_dtype);
     return fllm_check_launch("layernorm");
+}
+
+extern "C" int fllm_layernorm_conv(const float *x, const float *w1, float eps1, const float *conv, int taps, void *state, const int32_t *row_seg,
+                                   const int32_t *slots, void *out1, const float *w2, float eps2, void *out2, int rows, int width, int out_dtype,
+                                   hipStream_t stream) {
+    FLLM_REQUIRE(rows >= 0 && width > 0 && width <= 32 * kBlock && taps >= 1 && taps - 1 <= kMaxKeep, "layernorm_conv: bad sizes");
+    FLLM_REQUIRE(x && w1 && conv && (state || taps == 1) && row_seg && slots && out1 && ((w2 == nullptr) == (out2 == nullptr)) && eps1 > 0.f &&
+                     (w2 == nullptr || eps2 > 0.f), "layernorm_conv: operands missing");
+    if (rows == 0) return 0;
+    const dim3 grid(rows, (width + kBlock - 1) / kBlock);
+#define FLLM_LNC(T, N)                                                                                                                       \
+    hipLaunchKernelGGL((layernorm_conv_kernel<T, N>), grid, dim3(kBlock), 0, stream, x, w1, eps1, conv, taps, (T *)state, row_seg, slots,      \
+                       (T *)out1, w2, eps2, (T *)out2, width)
+#define FLLM_LNC_N(T)                                       \
+    do {                                                    \
+        if (width <= 4 * kBlock) FLLM_LNC(T, 4);            \
+        else if (width <= 8 * kBlock) FLLM_LNC(T, 8);       \
+        else FLLM_LNC(T, 32);                               \
+    } while (0)
+    if (out_dtype == FLLM_F32) FLLM_LNC_N(float);
+    else if (out_dtype == FLLM_BF16) FLLM_LNC_N(bf16_t);
+    else FLLM_REQUIRE(false, "layernorm_conv: unknown dtype %d", out_dtype);
+#undef FLLM_LNC_N
+#undef FLLM_LNC
+    return fllm_check_launch("layernorm_conv");
+}
+
+// 0: launched; negative: error; 1: declined (more than 8 rows, a width that is no multiple of 8)
+extern "C" int fllm_side_gate(const float *x, const void *w, const int32_t *ids, const void *table, int vocab, int table_width, int offset, void *out,
+                              int rows, int width, int dim, int dtype, hipStream_t stream) {
+    FLLM_REQUIRE(rows >= 0 && width > 0 && dim > 0 && vocab > 0 && offset >= 0 && offset + dim <= table_width, "side_gate: bad sizes");
+    FLLM_REQUIRE(x && w && ids && table && out, "side_gate: operands missing");
+    if (rows == 0) return 0;
+    if (rows > 8 || width % 8 != 0 || (((uintptr_t)x | (uintptr_t)w) & 15) != 0) return 1;
+#define FLLM_SIDE(T, R)                                                                                                                      \
+    hipLaunchKernelGGL((side_gate_kernel<T, R>), dim3(dim), dim3(kBlock), 0, stream, x, (const T *)w, ids, (const T *)table, vocab, table_width, \
+                       offset, (T *)out, rows, width, dim)
+#define FLLM_SIDE_R(T)                            \
+    do {                                          \
+        if (rows == 1) FLLM_SIDE(T, 1);           \
+        else if (rows == 2) FLLM_SIDE(T, 2);      \
+        else if (rows <= 4) FLLM_SIDE(T, 4);      \
+        else FLLM_SIDE(T, 8);                     \
+    } while (0)
+    if (dtype == FLLM_F32) FLLM_SIDE_R(float);
+    else if (dtype == FLLM_BF16) FLLM_SIDE_R(bf16_t);
+    else FLLM_REQUIRE(false, "side_gate: unknown dtype %d", dtype);
+#undef FLLM_SIDE_R
+#undef FLLM_SIDE
+    return fllm_check_launch("side_gate");
 }
 
 extern "C" int fllm_normed_pair_sum(float *out, const float *x, const float *wx, float a, const float *y, const float *wy, float b, float eps,

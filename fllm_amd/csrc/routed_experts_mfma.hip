@@ -81,7 +81,8 @@ scaled_rows_kernel(const bf16_t *__restrict__ h, int ldh, const float *__restric
     }
 }
 
-// MODE 0: act[pair, c] = a(g) * (u + up_offset) for 64 columns c a workgroup; A rows = the scaled rows in slot order;
+// MODE 0: act[pair, c] = a(g) * (u + up_offset) for 64 columns c a workgroup; A rows = the scaled rows in slot order (top 0), or the
+//         rows h[pair / top] as they are (top > 0: the picks' weights wait for the outputs);
 //         B = 64 gate rows and 64 up rows of the expert.  w: [E][2 N][K].
 // MODE 1: out[pair, c] = w[e][c] . act[pair] for GN columns, float32.  w: [E][N][K].
 // MODE 2: act[pair, c] = relu(w[e][c] . h[pair / top])^2 for GN columns: the up product of experts without a gate, whose rows
@@ -96,7 +97,7 @@ grouped_tiles_kernel(const bf16_t *__restrict__ x, int ldx, const int32_t *__res
                      float limit, float alpha, float up_offset, int k_per, size_t slice_stride, int top) {
     __shared__ __attribute__((aligned(16))) bf16_t As[GM * LDT];
     __shared__ __attribute__((aligned(16))) bf16_t Bs[GN * LDT];
-    __shared__ int s_pair[GM];
+    __shared__ int s_pair[GM], s_from[GM];      // a tile row's pair and the row of x that it reads (-1: none)
     static_assert(MODE != 0 || GN == 128, "gate and up rows come as 64 and 64");
     const int t = blockIdx.x % max_tiles, tn = blockIdx.x / max_tiles;     // neighbouring workgroups share a column tile
     if (t >= work[0]) return;
@@ -107,6 +108,8 @@ grouped_tiles_kernel(const bf16_t *__restrict__ x, int ldx, const int32_t *__res
     if (threadIdx.x < GM) {
         const int pair = threadIdx.x < count ? order[first + threadIdx.x] : -1;
         s_pair[threadIdx.x] = pair;
+        // MODE 1 reads the activations, which lie in pair order
+        s_from[threadIdx.x] = pair < 0 ? -1 : (MODE == 1 ? pair : (top > 0 ? pair / top : first + (int)threadIdx.x));
     }
     __syncthreads();
     const bf16_t *wb = w + (size_t)e * (MODE == 0 ? 2 : 1) * N * K;
@@ -135,10 +138,8 @@ grouped_tiles_kernel(const bf16_t *__restrict__ x, int ldx, const int32_t *__res
         for (int c = 0; c < kA; c++) {
             const int chunk = threadIdx.x + c * kThreads;
             const int row = chunk / (GK / 8), k = k0 + (chunk % (GK / 8)) * 8;
-            const int pair = s_pair[row];
-            // MODE 0 reads the scaled rows, which lie in slot order; MODE 1 the activations, which lie in pair order
-            const size_t from = MODE == 0 ? first + row : (MODE == 2 ? (pair < 0 ? 0 : pair / top) : pair);
-            ra[c] = (pair >= 0 && k < k_end) ? *(const bf16x8_t *)(x + from * ldx + k) : zero8();
+            const int from = s_from[row];
+            ra[c] = (from >= 0 && k < k_end) ? *(const bf16x8_t *)(x + (size_t)from * ldx + k) : zero8();
         }
 #pragma unroll
         for (int c = 0; c < kB; c++) {
@@ -249,13 +250,13 @@ extern "C" size_t fllm_experts_grouped_work_ints(int pairs, int E) {
 }
 
 // 0: launched, negative: error, 1: shape declined (the caller runs the plain kernels).  h bfloat16 [rows, K] (row stride ldh);
-// ids / weights [rows, top]; w_gate_up [E][2 inter][K]; w_down [E][N][inter]; act bfloat16 [rows * top, inter] and xs bfloat16
+// ids / weights [rows, top] (weights null: all 1, and no scaled copies of the rows are made); w_gate_up [E][2 inter][K]; w_down [E][N][inter]; act bfloat16 [rows * top, inter] and xs bfloat16
 // [rows * top, K] (scratch); out float32 [rows * top, N]; work: fllm_experts_grouped_work_ints() int32.
 extern "C" int fllm_experts_grouped(const void *h, int ldh, const int32_t *ids, const float *weights, int rows, int top,
                                     const void *w_gate_up, const void *w_down, int E, int inter, int K, int N, void *act, void *xs,
                                     float *out, int32_t *work, float *planes, float limit, float alpha, float up_offset, hipStream_t stream) {
     FLLM_REQUIRE(rows >= 0 && top > 0 && E > 0 && inter > 0 && K > 0 && N > 0 && ldh >= K, "experts_grouped: bad sizes");
-    FLLM_REQUIRE(h && ids && weights && w_gate_up && w_down && act && xs && out && work, "experts_grouped: operands missing");
+    FLLM_REQUIRE(h && ids && w_gate_up && w_down && act && (xs || !weights) && out && work, "experts_grouped: operands missing");
     if (!fllm_fast_kernels_enabled()) return 1;
     if (K % 8 != 0 || inter % 8 != 0 || ldh % 8 != 0 || E > 4096) return 1;
     if ((((uintptr_t)h | (uintptr_t)w_gate_up | (uintptr_t)w_down | (uintptr_t)act | (uintptr_t)xs) & 15) != 0) return 1;
@@ -273,16 +274,20 @@ extern "C" int fllm_experts_grouped(const void *h, int ldh, const int32_t *ids, 
     const long up_tiles = (inter + 63) / 64, down_tiles = (N + GN_DOWN - 1) / GN_DOWN;
     if (pairs > (1L << 24) || max_tiles * up_tiles > 0x7fffffffL || max_tiles * down_tiles > 0x7fffffffL) return 1;
     hipLaunchKernelGGL(group_pairs_kernel, dim3(1), dim3(1024), (size_t)3 * E * sizeof(int), stream, ids, (int)pairs, E, (int)max_tiles, GM, work);
-    hipLaunchKernelGGL(scaled_rows_kernel, dim3((unsigned)pairs), dim3(256), 0, stream, (const bf16_t *)h, ldh, weights, top,
-                       work + 1 + 3 * max_tiles, (bf16_t *)xs, K);
+    const bool scaled = weights != nullptr;
+    if (scaled)
+        hipLaunchKernelGGL(scaled_rows_kernel, dim3((unsigned)pairs), dim3(256), 0, stream, (const bf16_t *)h, ldh, weights, top,
+                           work + 1 + 3 * max_tiles, (bf16_t *)xs, K);
+    const void *up_in = scaled ? xs : h;
+    const int up_ld = scaled ? K : ldh;
     float *down_out = slices > 1 ? planes : out;
 #define FLLM_GROUPED(MODE, ROWS, COLS, X, LDX, W, NN, KK)                                                                                  \
     hipLaunchKernelGGL((grouped_tiles_kernel<MODE, ROWS, COLS>),                                                                           \
                        dim3((unsigned)(max_tiles * (MODE == 0 ? up_tiles : down_tiles)), MODE == 0 ? 1 : slices), dim3(kThreads), 0,        \
                        stream, (const bf16_t *)(X), LDX, work, (int)max_tiles, (const bf16_t *)(W), NN, KK, (bf16_t *)act, down_out, limit, \
-                       alpha, up_offset, MODE == 0 ? KK : k_per_down, (size_t)pairs * N, top)
-    if (GM == 128) FLLM_GROUPED(0, 128, 128, xs, K, w_gate_up, inter, K);
-    else FLLM_GROUPED(0, 64, 128, xs, K, w_gate_up, inter, K);
+                       alpha, up_offset, MODE == 0 ? KK : k_per_down, (size_t)pairs * N, scaled ? 0 : top)
+    if (GM == 128) FLLM_GROUPED(0, 128, 128, up_in, up_ld, w_gate_up, inter, K);
+    else FLLM_GROUPED(0, 64, 128, up_in, up_ld, w_gate_up, inter, K);
     if (GM == 128 && GN_DOWN == 128) FLLM_GROUPED(1, 128, 128, act, inter, w_down, N, inter);
     else if (GM == 128) FLLM_GROUPED(1, 128, 64, act, inter, w_down, N, inter);
     else if (GN_DOWN == 128) FLLM_GROUPED(1, 64, 128, act, inter, w_down, N, inter);

@@ -49,7 +49,7 @@ assert SAMPLE_ROW_BYTES == 32
 _lib = None
 
 
-ABI_VERSION = 18
+ABI_VERSION = 19
 
 
 def load_library(build_if_missing: bool = True):
@@ -153,6 +153,9 @@ def load_library(build_if_missing: bool = True):
         "fllm_cast_rows": [c_void, c_void, c_size, c_int, c_void],
         "fllm_softcap": [c_void, c_size, c_float, c_void],
         "fllm_gelu_side": [c_void, c_void, c_void, c_int, c_int, c_int, c_void, c_int, c_int, c_int, c_void],
+        "fllm_layernorm_conv": [c_void, c_void, c_float, c_void, c_int, c_void, c_void, c_void, c_void, c_void, c_float, c_void, c_int, c_int,
+                                c_int, c_void],
+        "fllm_side_gate": [c_void, c_void, c_void, c_void, c_int, c_int, c_int, c_void, c_int, c_int, c_int, c_int, c_void],
         "fllm_conv_qkv_store": [c_void, c_int, c_void, c_int, c_void, c_void, c_void, c_void, c_float, c_void, c_void, c_void, c_void, c_void,
                                 c_int, c_void, c_int, c_void, c_void, c_int, c_void, c_void, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
                                 c_int, c_int, c_int, c_int, c_int, c_void],
@@ -915,11 +918,11 @@ class Ops:
     GROUPED_EXPERTS_SHARE = 2      # and smaller ones that have this many pairs an expert: the plain kernels read an expert's
                                    # matrices once a pair, the grouped ones once a step
 
-    def experts_grouped(self, h: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor,
+    def experts_grouped(self, h: torch.Tensor, ids: torch.Tensor, weights: Optional[torch.Tensor], w_gate_up: torch.Tensor, w_down: torch.Tensor,
                         out: torch.Tensor, limit: float = 0.0, alpha: float = 1.0, up_offset: float = 0.0) -> bool:
         """`experts_gate_up` and `experts_down` in one call on the matrix cores (bfloat16, prompt portions): the pairs are
-        grouped by expert on the device, and an expert multiplies the rows that picked it as tiles.  out float32
-        [rows * top, width].  False: not taken (few rows, float32, sizes that are no multiples of 8), nothing was written."""
+        grouped by expert on the device, and an expert multiplies the rows that picked it as tiles.  weights None: all 1.
+        out float32 [rows * top, width].  False: not taken (few rows, float32, sizes that are no multiples of 8), nothing was written."""
         rows, K = h.shape
         top = ids.shape[1]
         E, two_i = w_gate_up.shape[0], w_gate_up.shape[1]
@@ -932,10 +935,12 @@ class Ops:
         _dense(w_gate_up, "w_gate_up", h.dtype, (E, two_i, K))
         _dense(w_down, "w_down", h.dtype, (E, N, two_i // 2))
         _dense(ids, "ids", torch.int32, (rows, top))
-        _dense(weights, "weights", torch.float32, (rows, top))
+        xs = None
+        if weights is not None:
+            _dense(weights, "weights", torch.float32, (rows, top))
+            xs = torch.empty((rows * top, K), dtype=h.dtype, device=h.device)      # the rows times their picks' weights
         _dense(out, "out", torch.float32, (rows * top, N))
         act = torch.empty((rows * top, two_i // 2), dtype=h.dtype, device=h.device)
-        xs = torch.empty((rows * top, K), dtype=h.dtype, device=h.device)      # the rows times their picks' weights
         work = torch.empty((int(self.lib.fllm_experts_grouped_work_ints(rows * top, E)),), dtype=torch.int32, device=h.device)
         need = int(self.lib.fllm_experts_grouped_plane_floats(rows * top, E, N, two_i // 2))     # a down product cut along K
         planes = torch.empty((need,), dtype=torch.float32, device=h.device) if need else None
@@ -990,6 +995,37 @@ class Ops:
         self._check(self.lib.fllm_norm_short_conv(_ptr(x), _ptr(norm_weight), float(eps), _ptr(w), _ptr(state), _ptr(row_seg), _ptr(slots),
                                                   _ptr(out), rows, width, taps, _DTYPE_CODE[out.dtype], self._stream()))
         return out
+
+    LAYERNORM_CONV_WIDTH = 8192      # widest rows whose values stay in registers between the sums and the outputs
+
+    def layernorm_conv(self, x: torch.Tensor, w1: torch.Tensor, eps1: float, conv: torch.Tensor, state: Optional[torch.Tensor],
+                       row_seg: torch.Tensor, slots: torch.Tensor, out1: torch.Tensor, w2: Optional[torch.Tensor] = None,
+                       eps2: Optional[float] = None, out2: Optional[torch.Tensor] = None) -> bool:
+        """`layernorm_pair`, the first norm through `short_conv`, in one kernel, for steps of ONE row a segment (segment s is row
+        s).  False: not taken (rows too wide), nothing was written."""
+        rows, width = x.shape
+        taps = conv.shape[1]
+        if width > self.LAYERNORM_CONV_WIDTH:
+            return False
+        _dense(x, "x", torch.float32)
+        _dense(w1, "w1", torch.float32, (width,))
+        _dense(conv, "conv", torch.float32, (width, taps))
+        _dense(out1, "out1", None, (rows, width))
+        _need(out1.dtype in _DTYPE_CODE, f"out dtype {out1.dtype} unsupported")
+        _need((w2 is None) == (out2 is None), "the second norm needs a weight and an output")
+        if w2 is not None:
+            _dense(w2, "w2", torch.float32, (width,))
+            _dense(out2, "out2", out1.dtype, (rows, width))
+        _dense(row_seg, "row_seg", torch.int32, (rows,))
+        _dense(slots, "slots", torch.int32)
+        _need(slots.numel() >= rows, "layernorm_conv: a slot a row")
+        if taps > 1:
+            _need(state is not None, "layernorm_conv: the taps before a step need a state")
+            _dense(state, "state", out1.dtype, (state.shape[0], taps - 1, width))
+        self._check(self.lib.fllm_layernorm_conv(_ptr(x), _ptr(w1), float(eps1), _ptr(conv), taps, _ptr(state), _ptr(row_seg), _ptr(slots),
+                                                 _ptr(out1), _ptr(w2), float(eps1 if eps2 is None else eps2), _ptr(out2), rows, width,
+                                                 _DTYPE_CODE[out1.dtype], self._stream()))
+        return True
 
     LINEAR_ATTENTION_PARTS_ROWS = 512      # steps of this many rows and more cut their segments into parts
 
@@ -1480,6 +1516,25 @@ class Ops:
         self._check(self.lib.fllm_gelu_side(_ptr(z), _ptr(ids), _ptr(table), table.shape[0], table.shape[1], int(offset), _ptr(out), rows, dim,
                                             _DTYPE_CODE[z.dtype], self._stream()))
         return out
+
+    def side_gate(self, x: torch.Tensor, w: torch.Tensor, ids: torch.Tensor, table: torch.Tensor, offset: int, out: torch.Tensor) -> bool:
+        """`gelu_side` of z = W x in one kernel, x the float32 rows of a stream.  False: not taken (more than 8 rows, a width that is no
+        multiple of 8), nothing was written."""
+        rows, width = x.shape
+        dim = w.shape[0]
+        _dense(x, "x", torch.float32)
+        _dense(w, "w", None, (dim, width))
+        _need(w.dtype in _DTYPE_CODE, f"dtype {w.dtype} unsupported")
+        _dense(ids, "ids", torch.int32, (rows,))
+        _dense(table, "table", w.dtype)
+        _need(table.dim() == 2 and 0 <= offset and offset + dim <= table.shape[1], "the table's rows are too short")
+        _dense(out, "out", w.dtype, (rows, dim))
+        code = self.lib.fllm_side_gate(_ptr(x), _ptr(w), _ptr(ids), _ptr(table), table.shape[0], table.shape[1], int(offset), _ptr(out), rows,
+                                       width, dim, _DTYPE_CODE[w.dtype], self._stream())
+        if code == 1:
+            return False
+        self._check(code)
+        return True
 
     def conv_qkv_store(self, joint: torch.Tensor, conv: torch.Tensor, bias: Optional[torch.Tensor], state: Optional[torch.Tensor],
                        q_weight: Optional[torch.Tensor], k_weight: Optional[torch.Tensor], eps: float, q_out: torch.Tensor,

@@ -117,16 +117,24 @@ class ParallelBlock(Block):
         # reader of the stream runs before the first sum into it
         project = getattr(self.mixer, "project_from_residual", None)
         projected = project(ctx, residual, self.mixer_norm) if project is not None else None
+        both = getattr(self.mixer, "convolved_norms", None)
         if self.feed_forward is None:
+            convolved = both(ctx, residual, self.mixer_norm, None, binding) if both is not None else None
             if projected is not None:
                 self.mixer.attend(ctx, projected, residual, binding)
+            elif convolved is not None:
+                self.mixer.forward_convolved(ctx, convolved[0], residual, binding)
             else:
                 self.mixer.forward(ctx, self.mixer_norm.forward(ctx, residual), residual, binding)
             return
         begin = getattr(self.feed_forward, "begin_from_residual", None)
         begun = begin(ctx, residual, self.feed_forward_norm) if begin is not None else None
-        h_mixer = h_ff = None
+        h_mixer = h_ff = convolved = None
         if projected is None and begun is None:
+            convolved = both(ctx, residual, self.mixer_norm, self.feed_forward_norm, binding) if both is not None else None
+        if convolved is not None:
+            h_mixer, h_ff = convolved          # one kernel, the mixer's input convolved on its way
+        elif projected is None and begun is None:
             first = getattr(self.mixer_norm, "row_form", lambda: None)()
             second = getattr(self.feed_forward_norm, "row_form", lambda: None)()
             if first is not None and second is not None and first[2] == second[2]:
@@ -140,6 +148,8 @@ class ParallelBlock(Block):
             h_ff = self.feed_forward_norm.forward(ctx, residual)
         if projected is not None:
             self.mixer.attend(ctx, projected, residual, binding)
+        elif convolved is not None:
+            self.mixer.forward_convolved(ctx, h_mixer, residual, binding)
         else:
             self.mixer.forward(ctx, h_mixer, residual, binding)
         if begun is not None:

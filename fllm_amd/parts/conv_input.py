@@ -100,6 +100,24 @@ class ConvInput(Mixer):
         self.inner.forward(ctx, out, residual, self._inner_binding(binding), **kw)
         return True
 
+    def convolved_norms(self, ctx, residual, norm, second, binding):
+        """Steps of one row a request behind layer norms: both norms of the row (the second may be None) and the convolution of
+        the first are one kernel.  (the wrapped mixer's input, the second norm's output), or None: not taken."""
+        rt = self.rt
+        fused = getattr(rt.ops, "layernorm_conv", None)
+        forms = [getattr(n, "row_form", lambda: None)() for n in (norm, second) if n is not None]
+        if fused is None or not ctx.uniform_rows or any(f is None or not f[2] for f in forms):
+            return None
+        h = rt.empty(tuple(residual.shape))
+        other = (forms[1][0], forms[1][1], rt.empty(tuple(residual.shape))) if second is not None else (None, None, None)
+        if not fused(residual, forms[0][0], forms[0][1], self.w, self._tail(binding), ctx.row_seg, ctx.slots, h, *other):
+            return None
+        return h, other[2]
+
+    def forward_convolved(self, ctx, h, residual, binding, **kw) -> None:
+        """`forward` of an input that the convolution has passed."""
+        self.inner.forward(ctx, h, residual, self._inner_binding(binding), **kw)
+
     @property
     def stores_branch(self):
         return bool(getattr(self.inner, "stores_branch", False))

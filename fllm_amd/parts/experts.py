@@ -119,7 +119,7 @@ class RoutedExperts(FeedForward):
         if self.weight_on == "output" and branch is not None:
             raise ValueError("experts whose weights lie on their outputs add to the stream themselves: no stored branch")
         if self.weight_on == "output":          # the experts read the rows as they are; the weights wait for the sum
-            on_output, weights = weights, self._ones(("ones", rows, self.top), (rows, self.top))
+            on_output, weights = weights, None
         parts = branch if branch is not None else rt.empty((rows * self.top, self.hidden), torch.float32)
         grouped = getattr(ops, "experts_grouped", None)
         if not self.gated:
@@ -130,6 +130,8 @@ class RoutedExperts(FeedForward):
                 ops.experts_down(act, ids, self.w_down, parts)
         elif grouped is None or not grouped(h, ids, weights, self.w_gate_up, self.w_down, parts, self.limit, self.alpha, self.up_offset):
             act = rt.empty((rows * self.top, self.inter))
+            if weights is None:
+                weights = self._ones(("ones", rows, self.top), (rows, self.top))
             ops.experts_gate_up(h, ids, weights, self.w_gate_up, act, self.limit, self.alpha, self.up_offset)
             ops.experts_down(act, ids, self.w_down, parts)
         if branch is None:

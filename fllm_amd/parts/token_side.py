@@ -38,12 +38,14 @@ class TokenSide(Part):
     def forward(self, ctx, x, embedding=None) -> None:
         rt, ops = self.rt, self.rt.ops
         rows = x.shape[0]
-        h = rt.empty((rows, self.size))
-        ops.cast_rows(x, h)
-        z = rt.empty((rows, self.dim))
-        ops.linear(h, self.w_gate, z)
         g = rt.empty((rows, self.dim))
-        ops.gelu_side(z, ctx.ids, self.table, self.offset, g)
+        gate = getattr(ops, "side_gate", None)          # steps of few rows: one kernel up to the gated numbers
+        if gate is None or not gate(x, self.w_gate, ctx.ids, self.table, self.offset, g):
+            h = rt.empty((rows, self.size))
+            ops.cast_rows(x, h)
+            z = rt.empty((rows, self.dim))
+            ops.linear(h, self.w_gate, z)
+            ops.gelu_side(z, ctx.ids, self.table, self.offset, g)
         y = rt.empty((rows, self.size), torch.float32)
         ops.linear(g, self.w_proj, y)
         ops.postnorm_add(x, y, self.weight, self.eps)

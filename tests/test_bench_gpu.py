@@ -121,6 +121,25 @@ def test_the_line_of_the_design_with_pooled_windows():
 
 
 @pytest.mark.gpu
+def test_the_line_of_the_design_with_gated_recurrences():
+    """`--design zoguzen`: chunked attention, minGRU and paired layers, all routed, beside Dumizen and Llama at equal sizes."""
+    done = run_bench("--design", "zoguzen", "--design-size", "small", "--layers", "4", "--steps", "6", "--warmup", "2",
+                     "--repeats", "1")
+    assert done.returncode == 0, done.stderr[-2000:]
+    lines = done.stdout.strip().splitlines()
+    assert len(lines) == 1
+    line = json.loads(lines[0])
+    assert line["sizes"]["layers"] == 4 and line["dtype"] == "bf16"
+    for model in ("zoguzen", "dumizen", "llama"):
+        got = line[model]
+        assert set(got) >= {"decode_b1", "decode_b8", "decode_b64", "prefill", "kernels"}
+        assert got["decode_b64"]["tokens_per_s"] > got["decode_b1"]["tokens_per_s"] > 0
+    prefill, decode = " ".join(line["zoguzen"]["kernels"]["prefill_us"]), " ".join(line["zoguzen"]["kernels"]["decode_b8_us"])
+    assert "masked_rows_kernel" in prefill and "gated_linear_chunked_kernel" in prefill and "grouped_tiles_kernel<0" in prefill
+    assert "masked_attention_kernel" not in prefill and "masked_heads_kernel" in decode and "layernorm_conv_kernel" in decode
+
+
+@pytest.mark.gpu
 def test_the_smoke_run_of_the_entry_file():
     """`__graft_entry__.smoke()` in a process of its own, as it is run: a few tokens of a tiny random model on the
     device against the plain implementation."""

@@ -104,6 +104,67 @@ def test_layer_norms_of_rows_with_an_offset(ops, ref, rows, width, dtype):
 
 
 @pytest.mark.parametrize("dtype", [F32, BF16])
+@pytest.mark.parametrize("two", [True, False])
+@pytest.mark.parametrize("width,taps", [(48, 2), (52, 1), (1024, 2), (1536, 4), (5000, 2)])
+def test_norms_and_convolution_in_one_kernel(ops, width, taps, two, dtype):
+    """Steps of single rows: the bits of layer norm and convolution one after the other, the state moved on likewise; a padding
+    row gives zeros and leaves the state alone."""
+    g = gen(width + taps)
+    rows = 5
+    x = (torch.randn(rows, width, generator=g) * 2 + 10.0).to(DEV)
+    w1, w2 = (1 + torch.rand(width, generator=g)).to(DEV), torch.randn(width, generator=g).to(DEV)
+    conv = torch.randn(width, taps, generator=g).to(DEV)
+    state = torch.randn(7, taps - 1, width, generator=g).to(dtype).to(DEV) if taps > 1 else None
+    slots, row_seg = torch.tensor([6, 0, 3, 1, 0], dtype=torch.int32, device=DEV), torch.tensor([0, 1, 2, 3, -1], dtype=torch.int32, device=DEV)
+    seg_start = torch.arange(rows + 1, dtype=torch.int32, device=DEV)
+    h, other, want = (torch.empty(rows, width, dtype=dtype, device=DEV) for _ in range(3))
+    ops.layernorm_pair(x, w1, 1e-5, h, w2, 1e-3, other)
+    st = None if state is None else state.clone()
+    ops.short_conv(h, conv, st, row_seg, seg_start, slots, want)
+    got, second = (torch.full((rows, width), float("nan"), dtype=dtype, device=DEV) for _ in range(2))
+    st2 = None if state is None else state.clone()
+    assert ops.layernorm_conv(x, w1, 1e-5, conv, st2, row_seg, slots, got, *((w2, 1e-3, second) if two else ()))
+    assert torch.equal(got[:4], want[:4]) and not got[4].any()
+    if two:
+        assert torch.equal(second[:4], other[:4]) and not second[4].any()
+    if state is not None:
+        assert torch.equal(st, st2) and not torch.equal(st2[6], state[6])
+    assert not ops.layernorm_conv(torch.zeros(1, 8193, device=DEV), w1, 1e-5, torch.zeros(8193, taps, device=DEV), st2, row_seg, slots, got)
+
+
+@pytest.mark.parametrize("dtype", [F32, BF16])
+@pytest.mark.parametrize("rows,width,dim", [(1, 48, 5), (2, 1536, 192), (3, 520, 1), (8, 1024, 64)])
+def test_the_side_inputs_gate_in_one_kernel(ops, ref, rows, width, dim, dtype):
+    g = gen(rows)
+    x, w = torch.randn(rows, width, generator=g) * 3, (torch.randn(dim, width, generator=g) * width ** -0.5).to(dtype)
+    table = torch.randn(31, 3 * dim, generator=g).to(dtype)
+    ids = torch.randint(0, 31, (rows,), generator=g, dtype=torch.int32)
+    want, got = torch.empty(rows, dim, dtype=F64), torch.full((rows, dim), float("nan"), dtype=dtype, device=DEV)
+    ref.gelu_side(x.to(dtype).double() @ w.double().T, ids, table.double(), 2 * dim, want)
+    assert ops.side_gate(x.to(DEV), w.to(DEV), ids.to(DEV), table.to(DEV), 2 * dim, got)
+    close(got, want, *((1e-5, 1e-5) if dtype == F32 else (BF16_EPS, 1e-3)))
+    nine = torch.zeros(9, width, device=DEV)
+    assert not ops.side_gate(nine, w.to(DEV), torch.zeros(9, dtype=torch.int32, device=DEV), table.to(DEV), 0, torch.empty(9, dim, dtype=dtype, device=DEV))
+    odd = torch.zeros(1, 52, device=DEV)
+    assert not ops.side_gate(odd, torch.zeros(dim, 52, dtype=dtype, device=DEV), ids[:1].to(DEV), table.to(DEV), 0, got[:1])
+
+
+@pytest.mark.parametrize("rows,experts,top", [(9, 4, 2), (40, 8, 3), (700, 5, 2)])
+def test_grouped_experts_read_the_rows_as_they_are(ops, rows, experts, top):
+    """Without weights: the bits of weights that are all 1, also where the rows lie apart from each other."""
+    g = gen(rows)
+    wide = torch.randn(rows, 200, generator=g).to(BF16).to(DEV)
+    h = wide[:, :136]
+    w_gate_up = (torch.randn(experts, 2 * 48, 136, generator=g) * 136 ** -0.5).to(BF16).to(DEV)
+    w_down = (torch.randn(experts, 136, 48, generator=g) * 48 ** -0.5).to(BF16).to(DEV)
+    ids = torch.stack([torch.randperm(experts, generator=g)[:top] for _ in range(rows)]).to(torch.int32).to(DEV)
+    want, got = (torch.full((rows * top, 136), float("nan"), device=DEV) for _ in range(2))
+    assert ops.experts_grouped(h, ids, torch.ones(rows, top, device=DEV), w_gate_up, w_down, want)
+    assert ops.experts_grouped(h, ids, None, w_gate_up, w_down, got)
+    assert torch.equal(got, want)
+
+
+@pytest.mark.parametrize("dtype", [F32, BF16])
 def test_the_small_passes(ops, ref, dtype):
     g = gen(2)
     rows, width, dim, vocab = 13, 200, 24, 50
@@ -358,7 +419,7 @@ def test_min_recurrence_in_parts_and_single_rows(ops, ref, width, segments, dtyp
 # the engine
 # ---------------------------------------------------------------------------------------------
 LENGTHS = {"A": [5, 30, 61, 120], "B": [45, 83, 2], "C": [9, 50, 77], "D": [100, 37, 260]}
-TOL = {"float32": 2e-5, "bfloat16": 6e-2}
+TOL = {"float32": 2e-5, "bfloat16": 4e-2}
 
 
 @pytest.fixture(scope="module")
@@ -369,7 +430,11 @@ def models(tmp_path_factory):
     out = {}
     for name, cfg in zc.CONFIGS.items():
         for dtype in ("float32", "bfloat16"):
-            tensors = zc.weights(cfg, 30 + ord(name), decided_router=dtype == "bfloat16")
+            # A side input of few lanes is divided by its own size: where all of them are nearly zero, the logits follow the last bit
+            # of every sum before it.  float32 runs a seed under which no position is such a one, bfloat16 more lanes as well.
+            if dtype == "bfloat16":
+                cfg = dict(cfg, token_side={"dim": 16})
+            tensors = zc.weights(cfg, 32 + ord(name), decided_router=dtype == "bfloat16")
             folder = zc.write_model(str(tmp_path_factory.mktemp(f"zoguzen_{name}_{dtype}")), cfg, tensors)
             requests = {f"r{i}": zc.random_ids(n, cfg["vocab"], 100 * ord(name) + i) for i, n in enumerate(LENGTHS[name])}
             w64 = zc.to_float64(tensors)
@@ -495,6 +560,34 @@ def test_the_residual_stream_after_every_layer(models):
     assert len(seen) == len(want) == 4
     for got, ref_x in zip(seen, want):
         assert np.abs(got - ref_x).max() <= 1e-5 * np.abs(ref_x).max()
+
+
+def test_decode_steps_take_the_fused_forms_and_prompts_the_tile_kernels(models, monkeypatch):
+    """D in bfloat16: a decode step norms a row for both branches and shifts the mixer's input in one kernel, gates the side input in
+    another, and runs no norm of its own but the model's last; a prompt's experts go to the matrix cores grouped by expert."""
+    from fllm_amd.engine import StepEntry
+    from fllm_amd.kernels import Ops
+    folder, cfg, requests, _, _ = models["D", "bfloat16"]
+    runner = make_runner(folder, "bfloat16", 16, 256, use_graphs=False)
+    kinds = [layer["type"] for layer in cfg["layers"]]
+    pairs, chunks, grus = (kinds.count(k) for k in ("parallel", "attention", "mingru"))
+    routed = sum(1 for layer in cfg["layers"] if layer["mlp"])
+    calls = []
+    for name in ("layernorm", "layernorm_pair", "layernorm_conv", "short_conv", "side_gate", "gelu_side", "cast_rows", "conv_qkv_store",
+                 "masked_attention", "gated_linear_attention", "min_recurrence", "normed_pair_sum", "experts_grouped", "experts_gate_up"):
+        inner = getattr(Ops, name)
+        monkeypatch.setattr(Ops, name, lambda self, *a, _n=name, _i=inner, **k: (calls.append(_n), _i(self, *a, **k))[1])
+    toks = requests["r0"]
+    runner.step([StepEntry("a", toks[:40], [])])
+    assert calls.count("layernorm_pair") == routed and calls.count("short_conv") == len(kinds) and calls.count("layernorm_conv") == 0
+    assert calls.count("experts_grouped") == routed and calls.count("experts_gate_up") == 0 and calls.count("gelu_side") == len(kinds)
+    assert calls.count("conv_qkv_store") == calls.count("masked_attention") == pairs + chunks
+    assert calls.count("gated_linear_attention") == calls.count("normed_pair_sum") == pairs and calls.count("min_recurrence") == grus
+    calls.clear()
+    runner.step([StepEntry("a", toks[40:41], [0])])
+    assert calls.count("layernorm_conv") == calls.count("side_gate") == len(kinds)
+    assert calls.count("layernorm") == 1 and not set(calls) & {"layernorm_pair", "short_conv", "cast_rows", "gelu_side"}
+    assert calls.count("conv_qkv_store") == calls.count("masked_attention") == pairs + chunks
 
 
 @pytest.mark.parametrize("name", ["A", "D"])
