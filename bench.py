@@ -319,9 +319,9 @@ def llama_config_of(size, layer_runs):
 
 
 def design_run(args):
-    """Prefill and decode throughput of another design (Menitar, Purivik, Venadra, Dumizen, Zoguzen) beside Llama at equal sizes (width, heads, head
-    size, feed-forward, vocabulary, as many layers as the other has layer runs), random bfloat16 weights, with the device
-    time of the kernels of a decode step and of a prefill step of each.  Prints one JSON line of its own."""
+    """Prefill and decode throughput of another design (Menitar, Purivik, Venadra, Dumizen, Zoguzen) beside Llama at equal sizes
+    (width, heads, head size, feed-forward, vocabulary, as many layers as the other has layer runs), random bfloat16 weights,
+    with the device time of the kernels of a decode step and of a prefill step of each.  Prints one JSON line of its own."""
     import gc
     import numpy as np
     import torch
